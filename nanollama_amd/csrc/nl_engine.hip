@@ -36,8 +36,6 @@
 #include <thread>
 #include <vector>
 
-namespace { void samp_free(nl::SampScratch &s); }
-
 using namespace nl;
 
 namespace {
@@ -3334,66 +3332,9 @@ int nl_decode_greedy(nl_handle e, int stream, int token, int pos, int n_steps, i
 
 namespace {
 
-// ---- on-device sampling ----------------------------------------------------
-// lane chunk of the select kernel: a multiple of 32 covering vocab / 1024 (vocab <= 131072)
-inline int samp_chunk(int vocab) { return ((vocab + SAMP_THREADS - 1) / SAMP_THREADS + 31) / 32 * 32; }
-
-hipError_t samp_alloc(SampScratch &s, int vocab, int n_uniforms) {
-    hipError_t rc;
-    if (samp_chunk(vocab) > 128) return hipErrorInvalidValue;   // vocab > 131072
-    const int nblocks = (vocab + 255) / 256;
-#define SA(ptr, count) if ((rc = hipMalloc((void **)&(ptr), (size_t)(count) * 4)) != hipSuccess) return rc
-    SA(s.keys_in, SAMP_THREADS * samp_chunk(vocab));   // (whole lane chunks: the select kernels load past vocab and mask)
-    if ((rc = hipMemset(s.keys_in, 0, (size_t)SAMP_THREADS * samp_chunk(vocab) * 4)) != hipSuccess) return rc;
-    SA(s.scal, 4); SA(s.pmax, nblocks); SA(s.h1g, 2 * 2048);
-    if ((rc = hipMemset(s.h1g, 0, 2048 * 8)) != hipSuccess) return rc;
-    SA(s.uniforms, std::max(n_uniforms, 1)); SA(s.recent, SAMP_THREADS); SA(s.recent_n, 1);
-#undef SA
-    return hipSuccess;
-}
-
-void samp_free(SampScratch &s) {
-    void *p[] = {s.keys_in, s.scal, s.pmax, s.h1g, s.uniforms, s.recent, s.recent_n};
-    for (void *q : p) if (q) (void)hipFree(q);
-    s = SampScratch{};
-}
-
-// one sampling decision on `logits` (device); advances ctl / ids / the recent window
-hipError_t launch_sample(const SampScratch &s, float *logits, int vocab, const nl_sample_params &p, int *ctl, int *ids,
-                         hipStream_t st, const EmbedParams *emb = nullptr) {
-    SampleParams P{};
-    if (emb) { P.embed = 1; P.emb = *emb; }
-    P.logits = logits; P.vocab = vocab; P.temp = p.temperature; P.top_p = p.top_p; P.top_k = std::max(p.top_k, 1);
-    P.rep_penalty = p.rep_penalty; P.recent = s.recent; P.recent_n = s.recent_n; P.rep_window = p.rep_window;
-    P.uniforms = s.uniforms; P.ctl = ctl; P.ids = ids;
-    P.keys_in = s.keys_in;
-    P.scal = s.scal; P.pmax = s.pmax; P.nblocks = (vocab + 255) / 256;
-    P.h1g = s.h1g; P.nblocks_pen = P.nblocks;
-    // Three selections, none with a sort (nl_sample.h): temp <= 0 -> argmax of the penalised logits; top_p < 1 -> sampleTopP by
-    // weighted radix selection (<= 32768 candidates in the registers of the one workgroup, up to 131072 streamed out of L2);
-    // otherwise sampleTopK by a 2-bit-per-pass selection of the k-th largest logit + a bitonic network over the <= 1024 candidates
-    P.radix = p.temperature > 0.f && p.top_p < 1.0f ? 1 : 0;
-    hipLaunchKernelGGL(samp_penalty_kernel, dim3(P.nblocks), dim3(256), 0, st, P);
-    if (P.radix) {
-        hipLaunchKernelGGL(samp_prob_hist_kernel, dim3((vocab + SAMP_THREADS - 1) / SAMP_THREADS), dim3(SAMP_THREADS), 0, st, P);
-        if (samp_chunk(vocab) == 32) hipLaunchKernelGGL(samp_select_radix_kernel<32>, dim3(1), dim3(SAMP_THREADS), 0, st, P);
-        else hipLaunchKernelGGL(samp_select_radix_stream_kernel, dim3(1), dim3(SAMP_THREADS), 0, st, P);
-    } else if (p.temperature > 0.f) {
-        if (samp_chunk(vocab) == 32) hipLaunchKernelGGL(samp_topk_kernel<false>, dim3(1), dim3(SAMP_THREADS), 0, st, P);
-        else hipLaunchKernelGGL(samp_topk_kernel<true>, dim3(1), dim3(SAMP_THREADS), 0, st, P);
-    } else {
-        hipLaunchKernelGGL(samp_argmax_select_kernel, dim3(1), dim3(SAMP_THREADS), 0, st, P);
-    }
-    return hipGetLastError();
-}
-
 int check_sample_params(nl_engine *e, const nl_sample_params *p) {
     auto bad = [&](const char *m) { return e ? e->fail(NL_ERR_INVALID, "%s", m) : (int)NL_ERR_INVALID; };
-    if (!p) return bad("sample params missing");
-    if (p->rep_window < 0 || p->rep_window > SAMP_THREADS) return bad("rep_window must be in [0, 1024] for on-device sampling");
-    if (!(p->top_p > 0.f)) return bad("top_p must be > 0");
-    if (p->top_k < 1 && p->top_p >= 1.f && p->temperature > 0.f) return bad("top_k must be >= 1");
-    if (p->top_k > SAMP_THREADS && p->top_p >= 1.f && p->temperature > 0.f) return bad("top_k must be <= 1024 for on-device sampling (the host loop takes larger lists)");
+    if (const char *m = sample_params_error(p)) return bad(m);
     return NL_OK;
 }
 
