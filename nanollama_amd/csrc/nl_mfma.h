@@ -1,0 +1,395 @@
+// nl_mfma.h -- dense matrix products of the layer-stack models (nl_stack.hip): weights and activations in MFMA operand order,
+// two element types behind one source.
+//
+//   T = __bf16 : v_mfma_f32_16x16x32_bf16, 32-bit accumulation
+//   T = float  : v_mfma_f32_16x16x4_f32, eight of them in place of one: IEEE single-precision products and sums
+//
+// OPERAND ORDER.  A matrix [rows][K] is cut into tiles of 16 rows x 32 columns; a tile is 64 runs of 8 elements, run
+// l = (k % 32) / 8 * 16 + row % 16, tiles of a row group one behind the other.  A wavefront's fragment is therefore one contiguous
+// 1 KiB (2 KiB for float) read in lane order, from HBM, L2 or LDS alike, and LDS-DMA copies tiles without touching registers.
+// Rows and K are padded with zeros to whole tiles.  Weights [out][in] are the A operand (rows = outputs), activations
+// [token][in] the B operand (rows = tokens); the accumulator of a 16 x 16 tile has D[row = 4 (lane / 16) + i][token = lane % 16],
+// so a lane ends up with four consecutive outputs of one token.
+//
+// Two kernels: many_kernel for prompts (a 128 x 128 tile per workgroup, LDS double buffer filled by LDS-DMA) and few_kernel for
+// decode batches of up to 64 tokens (one row tile per workgroup, K split over its wavefronts, the weights read once straight into
+// registers; for a handful of tokens the RMS norm of the layer's input runs in its prologue).  Epilogues: plain 32-bit store,
+// residual add (+ an optional second addend), gelu_tanh(gate) * up stored as the next product's operand.
+#pragma once
+#include "nl_kernels.h"
+
+namespace nl {
+
+typedef __bf16 bf16;
+typedef bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef bf16 bf16x4 __attribute__((ext_vector_type(4)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+constexpr int OPT = 512;          // elements of one operand tile (16 rows x 32 columns)
+enum { ST_F32 = 0, ST_RESID = 1, ST_GATED = 2 };   // epilogues
+
+template <typename T> struct Frag;
+template <> struct Frag<bf16> { bf16x8 v; };
+template <> struct Frag<float> { f32x4 a, b; };
+
+__device__ __forceinline__ void frag_zero(Frag<bf16> &f) { f.v = bf16x8{}; }
+__device__ __forceinline__ void frag_zero(Frag<float> &f) { f.a = f32x4{}; f.b = f32x4{}; }
+__device__ __forceinline__ float frag_get(const Frag<bf16> &f, int j) { return (float)f.v[j]; }
+__device__ __forceinline__ float frag_get(const Frag<float> &f, int j) { return j < 4 ? f.a[j & 3] : f.b[j & 3]; }
+__device__ __forceinline__ void frag_set(Frag<bf16> &f, int j, float x) { f.v[j] = (bf16)x; }
+__device__ __forceinline__ void frag_set(Frag<float> &f, int j, float x) { if (j < 4) f.a[j & 3] = x; else f.b[j & 3] = x; }
+
+__device__ __forceinline__ f32x4 mma(const Frag<bf16> &A, const Frag<bf16> &B, f32x4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(A.v, B.v, c, 0, 0, 0);
+}
+// the K order inside a fragment is the same permutation on both sides: step j multiplies element j of every lane's run
+__device__ __forceinline__ f32x4 mma(const Frag<float> &A, const Frag<float> &B, f32x4 c) {
+#pragma unroll
+    for (int j = 0; j < 4; j++) c = __builtin_amdgcn_mfma_f32_16x16x4f32(A.a[j], B.a[j], c, 0, 0, 0);
+#pragma unroll
+    for (int j = 0; j < 4; j++) c = __builtin_amdgcn_mfma_f32_16x16x4f32(A.b[j], B.b[j], c, 0, 0, 0);
+    return c;
+}
+
+// index of element (row, k) of an operand with nks tiles per row group
+__host__ __device__ inline long long op_index(int row, int k, int nks) {
+    return (((long long)(row >> 4) * nks + (k >> 5)) * 64 + ((k & 31) >> 3) * 16 + (row & 15)) * 8 + (k & 7);
+}
+__device__ __forceinline__ void put(bf16 *p, float v) { *p = (bf16)v; }
+__device__ __forceinline__ void put(float *p, float v) { *p = v; }
+__device__ __forceinline__ void put4(bf16 *p, f32x4 v) {
+    bf16x4 o;
+#pragma unroll
+    for (int i = 0; i < 4; i++) o[i] = (bf16)v[i];
+    *reinterpret_cast<bf16x4 *>(p) = o;
+}
+__device__ __forceinline__ void put4(float *p, f32x4 v) { *reinterpret_cast<f32x4 *>(p) = v; }
+
+__device__ __forceinline__ float sigmoid_f32(float z) {
+    const float e = expf(-fabsf(z));
+    return (z >= 0.f ? 1.f : e) / (1.f + e);
+}
+__device__ __forceinline__ float gelu_tanh_f32(float z) {
+    return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+__device__ __forceinline__ float wave_sum(float v) {
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
+    return v;
+}
+
+// 16 bytes per lane straight into LDS: lane i lands at lds_base + 16 i (lds_base wave-uniform)
+__device__ __forceinline__ void lds_dma16(const void *src_lane, void *lds_base) {
+    __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void *)src_lane,
+                                     (__attribute__((address_space(3))) void *)lds_base, 16, 0, 0);
+}
+__device__ __forceinline__ void lds_dma_wait() { asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); }
+
+// ------------------------------------------------------------- upload ---
+
+// rows x cols of a source matrix (bf16 bits or float) into operand order: row r goes to destination row
+// ((row0 + r) / 16 * tstride + toff) * 16 + (row0 + r) % 16, column c to k0 + c.  The destination was zeroed.
+template <typename T>
+__global__ void pack_operand_kernel(const void *src, int src_f32, long long rows, long long cols, T *dst, int nks, int row0, int k0,
+                                    int tstride, int toff) {
+    const long long n = rows * cols;
+    for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long long)gridDim.x * blockDim.x) {
+        const long long r = i / cols;
+        const int c = (int)(i - r * cols), R = row0 + (int)r;
+        const float v = src_f32 ? reinterpret_cast<const float *>(src)[i]
+                                : __uint_as_float((unsigned)reinterpret_cast<const unsigned short *>(src)[i] << 16);
+        put(dst + op_index(((R >> 4) * tstride + toff) * 16 + (R & 15), k0 + c, nks), v);
+    }
+}
+// a vector / small matrix as float, plus a constant (1 where a norm's gain is 1 + w)
+__global__ void widen_kernel(const void *src, int src_f32, long long n, float add, float *dst) {
+    for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long long)gridDim.x * blockDim.x)
+        dst[i] = (src_f32 ? reinterpret_cast<const float *>(src)[i]
+                          : __uint_as_float((unsigned)reinterpret_cast<const unsigned short *>(src)[i] << 16)) + add;
+}
+
+// ---------------------------------------------------- embedding, norm ---
+
+struct LookupParams {
+    const void *table;     // [vocab][dim] in operand order
+    const int *tok;
+    int nks, dim;
+    float scale;
+    float *x, *x0;         // x0 (may be null): a second copy for stacks that add the embedding output again
+};
+template <typename T>
+__global__ void __launch_bounds__(256) lookup_kernel(LookupParams P) {
+    const int n = blockIdx.x, token = P.tok[n];
+    for (int k = threadIdx.x; k < P.dim; k += 256) {
+        const float v = (float)reinterpret_cast<const T *>(P.table)[op_index(token, k, P.nks)] * P.scale;
+        P.x[(long long)n * P.dim + k] = v;
+        if (P.x0) P.x0[(long long)n * P.dim + k] = v;
+    }
+}
+
+// RMS norm of rows of the residual stream, stored as a product's operand (columns beyond dim zero)
+struct NormParams {
+    const float *x, *w;    // w: the factor itself
+    const int *rows;       // row of x for output token n; null: n
+    void *out;
+    int dim, nks;
+    float eps;
+};
+template <typename T>
+__global__ void __launch_bounds__(256) norm_operand_kernel(NormParams P) {
+    __shared__ float red[4];
+    const int n = blockIdx.x, tid = threadIdx.x;
+    const float *x = P.x + (long long)(P.rows ? P.rows[n] : n) * P.dim;
+    float ss = 0.f;
+    for (int k = tid; k < P.dim; k += 256) ss += x[k] * x[k];
+    ss = wave_sum(ss);
+    if ((tid & 63) == 0) red[tid >> 6] = ss;
+    __syncthreads();
+    const float inv = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)P.dim + P.eps);
+    T *out = reinterpret_cast<T *>(P.out);
+    for (int k8 = tid; k8 < P.nks * 4; k8 += 256) {
+        f32x4 a, b;
+#pragma unroll
+        for (int j = 0; j < 8; j++) {
+            const int k = k8 * 8 + j;
+            const float v = k < P.dim ? x[k] * inv * P.w[k] : 0.f;
+            if (j < 4) a[j] = v; else b[j - 4] = v;
+        }
+        T *o = out + op_index(n, k8 * 8, P.nks);
+        put4(o, a);
+        put4(o + 4, b);
+    }
+}
+
+// ----------------------------------------------------------- products ---
+
+struct MatParams {
+    const void *W;         // [nrt][nks] operand tiles; ST_GATED: gate tile, up tile, gate tile, ...
+    const void *X;         // [token tiles][nks]
+    int nks, nrt, n_tokens, rows;
+    float *out;            // ST_F32: [token][ldo]; ST_RESID: the residual stream, updated in place
+    int ldo;
+    const float *add2;     // ST_RESID: also added (same layout as out), or null
+    void *act;             // ST_GATED: [token tiles][act_nks] operand tiles
+    int act_nks;
+    // few_kernel with the norm in its prologue: B = norm(x)
+    const float *nx, *nw;
+    int ndim;
+    float neps;
+};
+
+__device__ __forceinline__ void store_rows(float *out, int ldo, int rows, int tok, int row, f32x4 v) {
+    float *o = out + (long long)tok * ldo + row;
+    if (row + 3 < rows && (ldo & 3) == 0) *reinterpret_cast<f32x4 *>(o) = v;
+    else
+        for (int i = 0; i < 4; i++)
+            if (row + i < rows) o[i] = v[i];
+}
+__device__ __forceinline__ void add_rows(float *out, const float *add2, int ldo, int rows, int tok, int row, f32x4 v) {
+    const long long at = (long long)tok * ldo + row;
+    if (row + 3 < rows && (ldo & 3) == 0) {
+        v += *reinterpret_cast<const f32x4 *>(out + at);
+        if (add2) v += *reinterpret_cast<const f32x4 *>(add2 + at);
+        *reinterpret_cast<f32x4 *>(out + at) = v;
+    } else
+        for (int i = 0; i < 4; i++)
+            if (row + i < rows) out[at + i] = out[at + i] + v[i] + (add2 ? add2[at + i] : 0.f);
+}
+// four consecutive feed-forward rows f16 * 16 + 4 g .. + 3 of one token
+template <typename T>
+__device__ __forceinline__ void store_gated(const MatParams &P, int tok, int f16, int g, f32x4 gate, f32x4 up) {
+    f32x4 v;
+#pragma unroll
+    for (int i = 0; i < 4; i++) v[i] = gelu_tanh_f32(gate[i]) * up[i];
+    put4(reinterpret_cast<T *>(P.act) + op_index(tok, f16 * 16 + 4 * g, P.act_nks), v);
+}
+
+// prompts: RTW row tiles x 4 token tiles per wavefront, 2 x 2 wavefronts
+template <typename T, int EPI, int RTW>
+__global__ void __launch_bounds__(256) many_kernel(MatParams P) {
+    constexpr int KS = sizeof(T) == 2 ? 2 : 1;             // k tiles per stage
+    constexpr int RT = 2 * RTW, NT = 8, UNIT = OPT * sizeof(T);
+    constexpr int STAGE = (RT + NT) * KS * UNIT;
+    extern __shared__ __align__(16) char lds[];
+    const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, g = lane >> 4;
+    const int nrb = (P.nrt + RT - 1) / RT, ntt = (P.n_tokens + 15) >> 4, ntb = (ntt + NT - 1) / NT, total = nrb * ntb;
+    // blocks b, b + 8, ... run on one XCD: give each XCD a contiguous range of (row block, token block), token blocks fastest, so
+    // that the token blocks of a row block share its weights in one L2
+    const int per = (total + 7) / 8, id = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+    if ((int)(blockIdx.x >> 3) >= per || id >= total) return;
+    const int rb = id / ntb, tb = id - rb * ntb;
+    const char *W = reinterpret_cast<const char *>(P.W), *X = reinterpret_cast<const char *>(P.X);
+    const int wr = w & 1, wt = w >> 1;
+    f32x4 acc[RTW][4] = {};
+    constexpr int NU = (RT + NT) * KS * (UNIT / 1024);     // 1 KiB pieces per stage
+    auto issue = [&](int ks0, int buf) {
+#pragma unroll
+        for (int u0 = 0; u0 < NU; u0 += 4) {
+            const int u = u0 + w, piece = u % (UNIT / 1024), tile = u / (UNIT / 1024), kk = tile % KS, t = tile / KS;
+            const int ks = min(ks0 + kk, P.nks - 1);
+            const char *src = t < RT ? W + ((long long)min(rb * RT + t, P.nrt - 1) * P.nks + ks) * UNIT
+                                     : X + ((long long)min(tb * NT + t - RT, ntt - 1) * P.nks + ks) * UNIT;
+            lds_dma16(src + piece * 1024 + lane * 16, lds + buf * STAGE + u * 1024);
+        }
+    };
+    issue(0, 0);
+    int buf = 0;
+    for (int ks0 = 0; ks0 < P.nks; ks0 += KS, buf ^= 1) {
+        lds_dma_wait();
+        __syncthreads();
+        if (ks0 + KS < P.nks) issue(ks0 + KS, buf ^ 1);
+        const char *base = lds + buf * STAGE;
+#pragma unroll
+        for (int kk = 0; kk < KS; kk++) {
+            if (KS > 1 && ks0 + kk >= P.nks) break;
+            Frag<T> b[4];
+#pragma unroll
+            for (int t = 0; t < 4; t++)
+                b[t] = *reinterpret_cast<const Frag<T> *>(base + ((RT + wt * 4 + t) * KS + kk) * UNIT + lane * sizeof(Frag<T>));
+#pragma unroll
+            for (int r = 0; r < RTW; r++) {
+                const Frag<T> a = *reinterpret_cast<const Frag<T> *>(base + ((wr * RTW + r) * KS + kk) * UNIT + lane * sizeof(Frag<T>));
+#pragma unroll
+                for (int t = 0; t < 4; t++) acc[r][t] = mma(a, b[t], acc[r][t]);
+            }
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < 4; t++) {
+        const int tok = (tb * NT + wt * 4 + t) * 16 + (lane & 15);
+        if (tok >= P.n_tokens) continue;
+#pragma unroll
+        for (int r = 0; r < RTW; r++) {
+            const int rt = rb * RT + wr * RTW + r;
+            if (rt >= P.nrt) continue;
+            const int row = rt * 16 + 4 * g;
+            if constexpr (EPI == ST_F32) store_rows(P.out, P.ldo, P.rows, tok, row, acc[r][t]);
+            else if constexpr (EPI == ST_RESID) add_rows(P.out, P.add2, P.ldo, P.rows, tok, row, acc[r][t]);
+            else if constexpr (RTW > 1) {
+                if ((r & 1) == 0) store_gated<T>(P, tok, rt >> 1, g, acc[r][t], acc[r + (RTW > 1 ? 1 : 0)][t]);
+            }
+        }
+    }
+}
+
+constexpr int FEW_MAX_TOKENS = 64;
+constexpr int FEW_NORM_ELEMS = 8192;      // tokens x dim up to which few_kernel computes the norm itself
+constexpr int FEW_PRE = 6;                // k tiles per wavefront and round: all their weight loads are in flight together
+
+// decode batches: one row tile (ST_GATED: a gate and an up tile) per workgroup, k tiles dealt to its wavefronts in turn
+template <typename T, int EPI, int NT, bool NORM>
+__global__ void __launch_bounds__(512) few_kernel(MatParams P) {
+    constexpr int RB = EPI == ST_GATED ? 2 : 1;
+    extern __shared__ __align__(16) char lds[];
+    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, nw = blockDim.x >> 6, g = lane >> 4, col = lane & 15;
+    const int rt = blockIdx.x * RB, nks = P.nks, n = P.n_tokens;
+    const Frag<T> *W = reinterpret_cast<const Frag<T> *>(P.W) + (long long)rt * nks * 64 + lane;
+    const Frag<T> *X = reinterpret_cast<const Frag<T> *>(P.X) + lane;
+    f32x4 acc[RB][NT] = {};
+    Frag<T> a[RB][FEW_PRE];
+    auto load_a = [&](int k0) {
+#pragma unroll
+        for (int u = 0; u < FEW_PRE; u++) {
+            const int ks = min(k0 + u * nw, nks - 1);
+#pragma unroll
+            for (int r = 0; r < RB; r++) a[r][u] = W[((long long)r * nks + ks) * 64];
+        }
+    };
+    load_a(w);
+    T *xs = reinterpret_cast<T *>(lds);                    // NORM: [nks][4][n][8]
+    if constexpr (NORM) {
+        float *red = reinterpret_cast<float *>(lds + (size_t)nks * 32 * n * sizeof(T));
+        for (int t = 0; t < n; t++) {
+            const float *x = P.nx + (long long)t * P.ndim;
+            float ss = 0.f;
+            for (int k = tid; k < P.ndim; k += blockDim.x) ss += x[k] * x[k];
+            ss = wave_sum(ss);
+            if (lane == 0) red[t * 8 + w] = ss;
+        }
+        __syncthreads();
+        for (int t = 0; t < n; t++) {
+            const float *x = P.nx + (long long)t * P.ndim;
+            float ss = 0.f;
+            for (int q = 0; q < nw; q++) ss += red[t * 8 + q];
+            const float inv = 1.f / sqrtf(ss / (float)P.ndim + P.neps);
+            for (int k = tid; k < nks * 32; k += blockDim.x)
+                put(xs + ((k >> 3) * n + t) * 8 + (k & 7), k < P.ndim ? x[k] * inv * P.nw[k] : 0.f);
+        }
+        __syncthreads();
+    }
+    for (int k0 = w; k0 < nks; k0 += FEW_PRE * nw) {
+        if (k0 != w) load_a(k0);
+#pragma unroll
+        for (int u = 0; u < FEW_PRE; u++) {
+            const int ks = k0 + u * nw;
+            if (ks >= nks) break;
+#pragma unroll
+            for (int t = 0; t < NT; t++) {
+                Frag<T> b;
+                frag_zero(b);
+                if (t * 16 + col < n) {
+                    if constexpr (NORM) b = *reinterpret_cast<const Frag<T> *>(xs + ((ks * 4 + g) * n + col) * 8);
+                    else b = X[((long long)t * nks + ks) * 64];
+                }
+#pragma unroll
+                for (int r = 0; r < RB; r++) acc[r][t] = mma(a[r][u], b, acc[r][t]);
+            }
+        }
+    }
+    // the wavefronts' partial tiles meet in LDS
+    __syncthreads();
+    f32x4 *red = reinterpret_cast<f32x4 *>(lds);           // [nw][RB * NT][64]
+#pragma unroll
+    for (int r = 0; r < RB; r++)
+#pragma unroll
+        for (int t = 0; t < NT; t++) red[(w * RB * NT + r * NT + t) * 64 + lane] = acc[r][t];
+    __syncthreads();
+    for (int i = tid; i < NT * 64; i += blockDim.x) {
+        const int t = i >> 6, l = i & 63, tok = t * 16 + (l & 15), row = rt * 16 + 4 * (l >> 4);
+        f32x4 v[RB] = {};
+        for (int q = 0; q < nw; q++)
+#pragma unroll
+            for (int r = 0; r < RB; r++) v[r] += red[(q * RB * NT + r * NT + t) * 64 + l];
+        if (tok >= n) continue;
+        if constexpr (EPI == ST_F32) store_rows(P.out, P.ldo, P.rows, tok, row, v[0]);
+        else if constexpr (EPI == ST_RESID) add_rows(P.out, P.add2, P.ldo, P.rows, tok, row, v[0]);
+        else store_gated<T>(P, tok, rt >> 1, l >> 4, v[0], v[RB - 1]);
+    }
+}
+
+template <typename T, int EPI, int NT, bool NORM>
+hipError_t launch_few_nt(const MatParams &P, hipStream_t st) {
+    const int RB = EPI == ST_GATED ? 2 : 1;
+    const int nw = NT > 2 ? 4 : 8;
+    size_t lds = (size_t)nw * RB * NT * 64 * 16;
+    if (NORM) lds = std::max(lds, (size_t)P.nks * 32 * P.n_tokens * sizeof(T) + (size_t)P.n_tokens * 8 * 4);
+    hipLaunchKernelGGL((few_kernel<T, EPI, NT, NORM>), dim3(P.nrt / RB), dim3(nw * 64), lds, st, P);
+    return hipGetLastError();
+}
+// is the norm of the product's input computed inside the launch?
+inline bool few_norm_ok(int n, int dim) { return n <= 16 && (long long)n * dim <= FEW_NORM_ELEMS; }
+
+template <typename T, int EPI>
+hipError_t launch_product(MatParams P, hipStream_t st, bool norm = false) {
+    if (P.n_tokens <= 0) return hipSuccess;
+    if (P.n_tokens <= FEW_MAX_TOKENS) {
+        if (norm) return launch_few_nt<T, EPI, 1, true>(P, st);
+        switch ((P.n_tokens + 15) / 16) {
+        case 1: return launch_few_nt<T, EPI, 1, false>(P, st);
+        case 2: return launch_few_nt<T, EPI, 2, false>(P, st);
+        case 3: return launch_few_nt<T, EPI, 3, false>(P, st);
+        default: return launch_few_nt<T, EPI, 4, false>(P, st);
+        }
+    }
+    const int ntb = (P.n_tokens + 127) / 128;
+    auto go = [&](auto kfn, int rt) {
+        const int total = (P.nrt + rt - 1) / rt * ntb;
+        const size_t lds = 2 * (size_t)(rt + 8) * (sizeof(T) == 2 ? 2 : 1) * OPT * sizeof(T);     // 48 or 64 KB
+        hipLaunchKernelGGL(kfn, dim3((total + 7) / 8 * 8), dim3(256), lds, st, P);
+        return hipGetLastError();
+    };
+    if ((P.nrt + 7) / 8 * ntb >= 512) return go(many_kernel<T, EPI, 4>, 8);
+    return go(many_kernel<T, EPI, 2>, 4);
+}
+
+}  // namespace nl

@@ -1,0 +1,377 @@
+// nl_winattn.h -- grouped-query softmax attention of the layer-stack models: optional per-head RMS norm of queries and keys, a
+// linear distance bias slope_h (i - j), an optional sliding window (keys i - window < j <= i), an output gate
+// sigmoid(g); query / key and value sizes may differ.  Scores, softmax and the norms are 32-bit; keys, values and the softmax
+// weights are operands of element type T (nl_mfma.h).
+//
+// CACHE.  A ring of R positions per (stream, kv head), position p in slot p % R, R a multiple of 64 and at least window - 1 + the
+// tokens a step may add, so that a step may write all its keys first and attend afterwards.  Both halves lie in MFMA operand
+// order, because both passes read them as the A operand:
+//   K  [R / 16][dim tiles of 32][64 lanes][8]       lane = dim-run * 16 + slot % 16                       (scores^T = K q^T)
+//   V  [R / 32][value tiles of 16][64 lanes][8]     lane = (slot % 16) / 4 * 16 + value % 16,
+//                                                   element j = slot / 16 % 2 * 4 + slot % 4              (out^T = V^T p^T)
+// The V order is the accumulator order of two 16-key score tiles, so the softmax weights become the second product's B operand
+// without leaving their lanes.  Reset is O(1): slots of another request are never visible (the mask is by position).
+//
+// PROMPTS: win_prep_kernel (norms, ring store, queries), win_attn_kernel (64 queries x one head per workgroup, keys and values
+// through LDS by LDS-DMA, double buffered).  DECODE: mix_decode_kernel -- attention heads (optionally split over key ranges, the
+// last split to arrive merges) and the linear-attention heads of a parallel layer in one launch.
+#pragma once
+#include "nl_linattn.h"
+
+namespace nl {
+
+constexpr int WA_Q = 64;                  // queries per workgroup
+constexpr int WA_MAX_DIM = 256;
+constexpr int WA_SPLIT_KEYS = 2048;       // keys one split of the decode launch can hold
+
+struct WinTile { int tok0, nq, pos0, stream; };       // queries [tok0, tok0 + nq) of the step, first one at position pos0
+
+struct WinParams {
+    const float *proj;          // [token][ldp]
+    int ldp, off_q, off_k, off_v, off_g;
+    int heads, kv_heads, dk, dv;
+    int nks, nvt;               // key tiles of 32, value tiles of 16
+    const float *qnorm, *knorm; // [dk] or null
+    float eps, scale, oscale;
+    const float *slope;         // [heads]
+    int window, R;              // window 0: everything
+    void *K, *V;                // this layer run, stream 0
+    long long kstride, vstride; // elements per stream
+    void *q;                    // [token][heads][nks * 32]
+    void *y;
+    int y_nks, y_k0;
+    const WinTile *tiles;
+    // token arrays (prompts: of the step, decode: of the batch)
+    const int *pos, *stream;
+    // decode
+    int nsplit;
+    float *part;                // [token][heads][nsplit][dv + 2]
+    unsigned *arrived;          // [token][heads], zero between launches
+};
+
+template <typename T> __device__ __forceinline__ T *ring_k(const WinParams &P, int stream, int g) {
+    return reinterpret_cast<T *>(P.K) + stream * P.kstride + (long long)g * P.R * P.nks * 32;
+}
+template <typename T> __device__ __forceinline__ T *ring_v(const WinParams &P, int stream, int g) {
+    return reinterpret_cast<T *>(P.V) + stream * P.vstride + (long long)g * P.R * P.nvt * 16;
+}
+__device__ __forceinline__ long long ring_k_at(int slot, int d, int nks) { return op_index(slot, d, nks); }
+__device__ __forceinline__ long long ring_v_at(int slot, int d, int nvt) {
+    return (((long long)(slot >> 5) * nvt + (d >> 4)) * 64 + ((slot & 15) >> 2) * 16 + (d & 15)) * 8 + ((slot & 31) >> 4) * 4 + (slot & 3);
+}
+
+// one wavefront per (token, head of q | k | v)
+template <typename T>
+__global__ void __launch_bounds__(256) win_prep_kernel(WinParams P) {
+    const int n = blockIdx.x, u = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (u >= P.heads + 2 * P.kv_heads) return;
+    const float *pr = P.proj + (long long)n * P.ldp;
+    if (u >= P.heads + P.kv_heads) {
+        const int g = u - P.heads - P.kv_heads, slot = P.pos[n] % P.R;
+        T *V = ring_v<T>(P, P.stream[n], g);
+        for (int d = lane; d < P.dv; d += 64) put(V + ring_v_at(slot, d, P.nvt), pr[P.off_v + g * P.dv + d]);
+        return;
+    }
+    const bool isq = u < P.heads;
+    const float *src = pr + (isq ? P.off_q + u * P.dk : P.off_k + (u - P.heads) * P.dk), *nw = isq ? P.qnorm : P.knorm;
+    float v[WA_MAX_DIM / 64], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < WA_MAX_DIM / 64; i++) {
+        v[i] = lane + 64 * i < P.dk ? src[lane + 64 * i] : 0.f;
+        ss += v[i] * v[i];
+    }
+    const float inv = nw ? 1.f / sqrtf(wave_sum(ss) / (float)P.dk + P.eps) : 1.f;
+    T *q = reinterpret_cast<T *>(P.q) + ((long long)n * P.heads + u) * P.nks * 32;
+    T *K = isq ? nullptr : ring_k<T>(P, P.stream[n], u - P.heads);
+    const int slot = isq ? 0 : P.pos[n] % P.R;
+#pragma unroll
+    for (int i = 0; i < WA_MAX_DIM / 64; i++) {
+        const int d = lane + 64 * i;
+        if (d >= P.nks * 32) break;
+        const float o = d < P.dk ? v[i] * inv * (nw ? nw[d] : 1.f) : 0.f;
+        if (isq) put(q + d, o);
+        else put(K + ring_k_at(slot, d, P.nks), o);
+    }
+}
+
+template <typename T> __device__ __forceinline__ float soft_exp(float x) { return sizeof(T) == 2 ? __expf(x) : expf(x); }
+
+// grid (tiles, heads); M bounds the key tiles (nks <= M) and value tiles (nvt <= 2 M)
+template <typename T, int M>
+__global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
+    constexpr int KT = sizeof(T) == 2 ? 64 : 32, UNIT = OPT * sizeof(T);
+    extern __shared__ __align__(16) char lds[];
+    const WinTile tl = P.tiles[blockIdx.x];
+    const int h = blockIdx.y, gk = h / (P.heads / P.kv_heads), tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, c = lane & 15;
+    const int nks = P.nks, nvt = P.nvt, qi = w * 16 + c, tok = tl.tok0 + min(qi, tl.nq - 1), qpos = tl.pos0 + min(qi, tl.nq - 1);
+    const int win = P.window > 0 ? P.window : 0x7fffffff;
+    Frag<T> qf[M];
+    {
+        const T *q = reinterpret_cast<const T *>(P.q) + ((long long)tok * P.heads + h) * nks * 32 + g * 8;
+#pragma unroll
+        for (int k = 0; k < M; k++)
+            if (k < nks) qf[k] = *reinterpret_cast<const Frag<T> *>(q + k * 32);
+    }
+    const char *K = reinterpret_cast<const char *>(ring_k<T>(P, tl.stream, gk)), *V = reinterpret_cast<const char *>(ring_v<T>(P, tl.stream, gk));
+    const int kpieces = KT / 16 * nks * (UNIT / 1024), vpieces = KT / 32 * nvt * (UNIT / 1024), stage = (kpieces + vpieces) * 1024;
+    const int jhi = tl.pos0 + tl.nq - 1, jlo = max(0, tl.pos0 - win + 1), j0 = jlo / KT * KT;
+    // queries of this wavefront: none of them sees keys outside [wlo, whi]
+    const int wq = min(w * 16, tl.nq - 1), whi = tl.pos0 + min(w * 16 + 15, tl.nq - 1), wlo = max(0, tl.pos0 + wq - win + 1);
+    auto issue = [&](int j, int buf) {
+        const int slot = j % P.R;                        // R is a multiple of KT: a tile of keys is one contiguous run
+        const char *ks = K + (long long)(slot >> 4) * nks * UNIT, *vs = V + (long long)(slot >> 5) * nvt * UNIT;
+        for (int u = w; u < kpieces + vpieces; u += 4)
+            lds_dma16((u < kpieces ? ks + u * 1024 : vs + (u - kpieces) * 1024) + lane * 16, lds + buf * stage + u * 1024);
+    };
+    f32x4 o[2 * M] = {};
+    float m = -INFINITY, l = 0.f;
+    const float slope = P.slope ? P.slope[h] : 0.f;
+    issue(j0, 0);
+    int buf = 0;
+    for (int j = j0; j <= jhi; j += KT, buf ^= 1) {
+        lds_dma_wait();
+        __syncthreads();
+        if (j + KT <= jhi) issue(j + KT, buf ^ 1);
+        if (j > whi || j + KT - 1 < wlo) continue;       // (every wavefront meets the barrier of every tile)
+        const char *kb = lds + buf * stage, *vb = kb + kpieces * 1024;
+        f32x4 s[KT / 16];
+        float mx = m;
+#pragma unroll
+        for (int a = 0; a < KT / 16; a++) {
+            s[a] = f32x4{};
+#pragma unroll
+            for (int k = 0; k < M; k++)
+                if (k < nks) s[a] = mma(*reinterpret_cast<const Frag<T> *>(kb + (a * nks + k) * UNIT + lane * sizeof(Frag<T>)), qf[k], s[a]);
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int dist = qpos - (j + a * 16 + 4 * g + i);
+                s[a][i] = dist >= 0 && dist < win ? s[a][i] * P.scale - slope * (float)dist : -INFINITY;
+                mx = fmaxf(mx, s[a][i]);
+            }
+        }
+        mx = fmaxf(mx, __shfl_xor(mx, 16));
+        mx = fmaxf(mx, __shfl_xor(mx, 32));
+        const float base = mx == -INFINITY ? 0.f : mx, corr = soft_exp<T>(m - base);
+        m = mx;
+        float add = 0.f;
+        Frag<T> p[KT / 32];
+#pragma unroll
+        for (int a = 0; a < KT / 16; a++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const float e = soft_exp<T>(s[a][i] - base);
+                add += e;
+                frag_set(p[a >> 1], (a & 1) * 4 + i, e);
+            }
+        l = l * corr + add;
+#pragma unroll
+        for (int t = 0; t < 2 * M; t++)
+            if (t < nvt) {
+                o[t] *= corr;
+#pragma unroll
+                for (int b = 0; b < KT / 32; b++)
+                    o[t] = mma(*reinterpret_cast<const Frag<T> *>(vb + (b * nvt + t) * UNIT + lane * sizeof(Frag<T>)), p[b], o[t]);
+            }
+    }
+    l += __shfl_xor(l, 16);
+    l += __shfl_xor(l, 32);
+    if (qi >= tl.nq) return;
+    const float inv = P.oscale / l;
+    T *y = reinterpret_cast<T *>(P.y);
+    const float *gz = P.proj + (long long)tok * P.ldp + P.off_g + h * P.dv;
+#pragma unroll
+    for (int t = 0; t < 2 * M; t++)
+        if (t < nvt) {
+            const int d = t * 16 + 4 * g, k = P.y_k0 + h * P.dv + d;
+            if (d + 3 < P.dv && (k & 3) == 0) {
+                f32x4 r;
+#pragma unroll
+                for (int i = 0; i < 4; i++) r[i] = o[t][i] * inv * (P.off_g < 0 ? 1.f : sigmoid_f32(gz[d + i]));
+                put4(y + op_index(tok, k, P.y_nks), r);
+            } else
+                for (int i = 0; i < 4; i++)
+                    if (d + i < P.dv) put(y + op_index(tok, k + i, P.y_nks), o[t][i] * inv * (P.off_g < 0 ? 1.f : sigmoid_f32(gz[d + i])));
+        }
+}
+
+// --------------------------------------------------------------- decode ---
+
+__host__ __device__ inline size_t win_decode_lds(int nks, int nvt) {
+    return (size_t)(2 * nks * 32 + 2 * nvt * 16 + WA_SPLIT_KEYS + 64 + 16) * 4;
+}
+
+// one (head, key split, token of the batch) by a workgroup of 256
+template <typename T>
+__device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int split, int n, int stream, int pos, char *lds) {
+    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, c = lane & 15, dk = P.dk, dv = P.dv, nks = P.nks, nvt = P.nvt;
+    const int gq = P.heads / P.kv_heads, gk = h / gq;
+    float *qn = reinterpret_cast<float *>(lds), *kn = qn + nks * 32, *vn = kn + nks * 32, *os = vn + nvt * 16, *sc = os + nvt * 16, *red = sc + WA_SPLIT_KEYS + 64;
+    const float *pr = P.proj + (long long)n * P.ldp;
+    const int win = P.window > 0 ? P.window : 0x7fffffff, lo = max(0, pos - win + 1);
+    // the split's blocks of 32 keys, at most WA_SPLIT_KEYS / 32 + 1 of them; the last block holds the new position
+    const int b0 = lo >> 5, nb = (pos >> 5) - b0 + 1, per = (nb + P.nsplit - 1) / P.nsplit, bf = b0 + split * per, bl = min(bf + per, b0 + nb);
+    const bool newest = bf < bl && bl == b0 + nb;
+    // wavefront 0 the query, wavefront 1 the new key, the others the new value
+    if (w < 2) {
+        const float *src = pr + (w == 0 ? P.off_q + h * dk : P.off_k + gk * dk), *nw = w == 0 ? P.qnorm : P.knorm;
+        float v[WA_MAX_DIM / 64], ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < WA_MAX_DIM / 64; i++) {
+            v[i] = lane + 64 * i < dk ? src[lane + 64 * i] : 0.f;
+            ss += v[i] * v[i];
+        }
+        const float inv = nw ? 1.f / sqrtf(wave_sum(ss) / (float)dk + P.eps) : 1.f;
+#pragma unroll
+        for (int i = 0; i < WA_MAX_DIM / 64; i++) {
+            const int d = lane + 64 * i;
+            if (d < nks * 32) (w == 0 ? qn : kn)[d] = d < dk ? v[i] * inv * (nw ? nw[d] : 1.f) : 0.f;
+        }
+    } else
+        for (int d = tid - 128; d < dv; d += 128) vn[d] = pr[P.off_v + gk * dv + d];
+    __syncthreads();
+    T *K = ring_k<T>(P, stream, gk), *V = ring_v<T>(P, stream, gk);
+    if (newest && h % gq == 0) {
+        const int slot = pos % P.R;
+        for (int d = tid; d < nks * 32; d += 256) put(K + ring_k_at(slot, d, nks), kn[d]);
+        for (int d = tid; d < dv; d += 256) put(V + ring_v_at(slot, d, nvt), vn[d]);
+    }
+    // scores: 16 keys per wavefront and round
+    const float slope = P.slope ? P.slope[h] : 0.f;
+    float mx = -INFINITY;
+    for (int t = 2 * bf + w; t < 2 * bl; t += 4) {
+        const int j = t * 16 + c;
+        const Frag<T> *kf = reinterpret_cast<const Frag<T> *>(K) + (long long)((t * 16) % P.R >> 4) * nks * 64 + lane;
+        float dot = 0.f;
+#pragma unroll 4
+        for (int k = 0; k < nks; k++) {
+            const Frag<T> f = kf[k * 64];
+            const f32x4 q0 = *reinterpret_cast<const f32x4 *>(qn + k * 32 + g * 8), q1 = *reinterpret_cast<const f32x4 *>(qn + k * 32 + g * 8 + 4);
+            if (j == pos) {      // (its ring slot may not be written yet)
+                const f32x4 k0 = *reinterpret_cast<const f32x4 *>(kn + k * 32 + g * 8), k1 = *reinterpret_cast<const f32x4 *>(kn + k * 32 + g * 8 + 4);
+#pragma unroll
+                for (int i = 0; i < 4; i++) dot = fmaf(k1[i], q1[i], fmaf(k0[i], q0[i], dot));
+            } else
+#pragma unroll
+                for (int i = 0; i < 4; i++) dot = fmaf(frag_get(f, 4 + i), q1[i], fmaf(frag_get(f, i), q0[i], dot));
+        }
+        dot += __shfl_xor(dot, 16);
+        dot += __shfl_xor(dot, 32);
+        const float s = j >= lo && j <= pos ? dot * P.scale - slope * (float)(pos - j) : -INFINITY;
+        if (g == 0) sc[j - bf * 32] = s;
+        mx = fmaxf(mx, s);
+    }
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
+    if (lane == 0) red[w] = mx;
+    __syncthreads();
+    mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+    const float base = mx == -INFINITY ? 0.f : mx;
+    float sum = 0.f;
+    for (int i = tid; i < (bl - bf) * 32; i += 256) {
+        const float e = expf(sc[i] - base);
+        sc[i] = e;
+        sum += e;
+    }
+    sum = wave_sum(sum);
+    if (lane == 0) red[4 + w] = sum;
+    __syncthreads();
+    sum = red[4] + red[5] + red[6] + red[7];
+    const float pnew = newest ? sc[pos - bf * 32] : 0.f;
+    // values: a wavefront per tile of 16, lane (value c, key group g)
+    for (int t = w; t < nvt; t += 4) {
+        float a = 0.f;
+#pragma unroll 4
+        for (int b = bf; b < bl; b++) {
+            const Frag<T> f = reinterpret_cast<const Frag<T> *>(V)[((long long)((b * 32) % P.R >> 5) * nvt + t) * 64 + lane];
+            const float *p = sc + (b - bf) * 32 + g * 4;
+            const int jb = b * 32 + g * 4;
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                // keys outside the window weigh 0; the new key's value comes from this step's projection, not from the ring
+                const float v0 = jb + i == pos ? 0.f : frag_get(f, i), v1 = jb + 16 + i == pos ? 0.f : frag_get(f, 4 + i);
+                a = fmaf(p[16 + i], v1, fmaf(p[i], v0, a));
+            }
+        }
+        a += __shfl_xor(a, 16);
+        a += __shfl_xor(a, 32);
+        if (g == 0) os[t * 16 + c] = t * 16 + c < dv ? a + (newest ? pnew * vn[t * 16 + c] : 0.f) : 0.f;
+    }
+    __syncthreads();
+    T *y = reinterpret_cast<T *>(P.y);
+    auto finish = [&](int d, float val) {
+        const float gate = P.off_g < 0 ? 1.f : sigmoid_f32(pr[P.off_g + h * dv + d]);
+        put(y + op_index(n, P.y_k0 + h * dv + d, P.y_nks), val * gate * P.oscale);
+    };
+    if (P.nsplit == 1) {
+        for (int d = tid; d < dv; d += 256) finish(d, os[d] / sum);
+        return;
+    }
+    // several splits: every one leaves (max, sum, unnormalised values); the last to arrive merges, nobody waits
+    float *mine = P.part + (((long long)n * P.heads + h) * P.nsplit + split) * (dv + 2);
+    for (int d = tid; d < dv; d += 256) __hip_atomic_store(mine + 2 + d, os[d], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    if (tid == 0) {
+        __hip_atomic_store(mine, mx, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        __hip_atomic_store(mine + 1, sum, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    }
+    __threadfence();
+    __syncthreads();
+    unsigned *arr = P.arrived + n * P.heads + h;
+    unsigned *last = reinterpret_cast<unsigned *>(red + 8);
+    if (tid == 0) *last = __hip_atomic_fetch_add(arr, 1u, __ATOMIC_ACQ_REL, __HIP_MEMORY_SCOPE_AGENT);
+    __syncthreads();
+    if (*last + 1 != (unsigned)P.nsplit) return;
+    __threadfence();
+    const float *all = P.part + ((long long)n * P.heads + h) * P.nsplit * (dv + 2);
+    auto rd = [&](int s, int i) { return __hip_atomic_load(all + (long long)s * (dv + 2) + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); };
+    float gm = -INFINITY;
+    for (int s = 0; s < P.nsplit; s++) gm = fmaxf(gm, rd(s, 0));
+    for (int d = tid; d < dv; d += 256) {
+        float a = 0.f, b = 0.f;
+        for (int s = 0; s < P.nsplit; s++) {
+            const float f = expf(rd(s, 0) - gm);
+            a += f * rd(s, 1);
+            b += f * rd(s, 2 + d);
+        }
+        finish(d, b / a);
+    }
+    if (tid == 0) __hip_atomic_store(arr, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+}
+
+// a decode batch's mixers: grid (attention heads x splits + linear-attention heads, tokens)
+template <typename T>
+__global__ void __launch_bounds__(256) mix_decode_kernel(WinParams A, GlaParams L) {
+    extern __shared__ __align__(16) char lds[];
+    const int n = blockIdx.y, pos = A.pos[n], stream = A.stream[n], na = A.heads * A.nsplit;
+    if ((int)blockIdx.x < na) win_decode_block<T>(A, blockIdx.x / A.nsplit, blockIdx.x % A.nsplit, n, stream, pos, lds);
+    else gla_decode_block<T>(L, blockIdx.x - na, n, stream, pos, lds);
+}
+
+template <typename T>
+hipError_t launch_mix_decode(const WinParams &A, const GlaParams &L, int n, hipStream_t st) {
+    size_t lds = 0;
+    if (A.heads) lds = win_decode_lds(A.nks, A.nvt);
+    if (L.heads) lds = std::max(lds, gla_decode_lds(L.dkp, L.dvp, L.rank));
+    hipLaunchKernelGGL(mix_decode_kernel<T>, dim3(A.heads * A.nsplit + L.heads, n), dim3(256), lds, st, A, L);
+    return hipGetLastError();
+}
+
+template <typename T>
+hipError_t launch_win_attn(const WinParams &P, int n_tokens, int ntiles, hipStream_t st) {
+    hipLaunchKernelGGL(win_prep_kernel<T>, dim3(n_tokens, (P.heads + 2 * P.kv_heads + 3) / 4), dim3(256), 0, st, P);
+    const size_t lds = 2 * (size_t)((sizeof(T) == 2 ? 4 : 2) * P.nks + (sizeof(T) == 2 ? 2 : 1) * P.nvt) * OPT * sizeof(T);
+    auto go = [&](auto kfn) {
+        // (more than 64 KB of LDS needs the attribute; cheap enough to set at every such launch)
+        if (lds > 65536)
+            if (hipError_t s = hipFuncSetAttribute(reinterpret_cast<const void *>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)) return s;
+        hipLaunchKernelGGL(kfn, dim3(ntiles, P.heads), dim3(256), lds, st, P);
+        return hipGetLastError();
+    };
+    const int m = std::max(P.nks, (P.nvt + 1) / 2);
+    if (m <= 1) return go(win_attn_kernel<T, 1>);
+    if (m <= 2) return go(win_attn_kernel<T, 2>);
+    if (m <= 3) return go(win_attn_kernel<T, 3>);
+    if (m <= 4) return go(win_attn_kernel<T, 4>);
+    return go(win_attn_kernel<T, 8>);
+}
+
+}  // namespace nl

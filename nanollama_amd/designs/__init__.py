@@ -1,0 +1,4 @@
+"""Designs of layer-stack models: architecture name of config.json -> function (config, tensor shape) -> StackSpec."""
+from .ganidra import ganidra_spec
+
+DESIGNS = {"Ganidra": ganidra_spec}

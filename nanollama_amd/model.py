@@ -54,29 +54,35 @@ class LlamaState:
         self.pos = 0
 
 
-class LlamaModel:
-    def __init__(self, config: LlamaConfig, handle, max_streams: int):
+class HipModel:
+    """A model behind the C ABI, whatever its family: what the generation loop, the batch scheduler, the CLI and the server call.
+    `config` needs vocab_size and seq_len; `L` is the family's library."""
+
+    def __init__(self, config, handle, max_streams: int, L):
         self.config = config
         self.state = LlamaState(config.vocab_size)
-        self.gamma = None  # go/model.go:23 (gamma injection is out of scope)
+        self.gamma = None  # go/model.go:23
         self._h = handle
+        self._L = L
         self.max_streams = max_streams
+
+    def _check(self, rc: int) -> None:
+        _lib.check(self._h, rc, self._L)
 
     # --- Forward go/model.go:490 ---
     def forward(self, token: int, pos: int, stream: int = 0) -> None:
-        L = _lib.lib()
-        _lib.check(self._h, L.nl_forward(self._h, stream, int(token), int(pos),
+        self._check(self._L.nl_forward(self._h, stream, int(token), int(pos),
                                          self.state.logits.ctypes.data_as(C.POINTER(C.c_float))))
 
     def forward_argmax(self, token: int, pos: int, stream: int = 0) -> int:
         out = C.c_int(0)
-        _lib.check(self._h, _lib.lib().nl_forward_argmax(self._h, stream, int(token), int(pos), C.byref(out)))
+        self._check(self._L.nl_forward_argmax(self._h, stream, int(token), int(pos), C.byref(out)))
         return out.value
 
     def decode_greedy(self, token: int, pos: int, n_steps: int, stream: int = 0) -> List[int]:
         ids = (C.c_int * max(n_steps, 1))()
         done = C.c_int(0)
-        _lib.check(self._h, _lib.lib().nl_decode_greedy(self._h, stream, int(token), int(pos), int(n_steps), ids,
+        self._check(self._L.nl_decode_greedy(self._h, stream, int(token), int(pos), int(n_steps), ids,
                                                         C.byref(done)))
         return [int(ids[i]) for i in range(done.value)]
 
@@ -93,7 +99,7 @@ class LlamaModel:
         nrec = C.c_int(len(recent))
         ids = (C.c_int * max(n_steps, 1))()
         done = C.c_int(0)
-        _lib.check(self._h, _lib.lib().nl_sample_decode(self._h, stream, int(pos), int(n_steps), C.byref(p),
+        self._check(self._L.nl_sample_decode(self._h, stream, int(pos), int(n_steps), C.byref(p),
                                                         u.ctypes.data_as(C.POINTER(C.c_float)), rec, C.byref(nrec), ids,
                                                         C.byref(done)))
         return [int(ids[i]) for i in range(done.value)], [int(rec[i]) for i in range(nrec.value)]
@@ -102,17 +108,84 @@ class LlamaModel:
         """The prompt loop of Generate (go/main.go:160-166) queued on the device in one call."""
         arr = (C.c_int * len(tokens))(*[int(t) for t in tokens])
         out = self.state.logits.ctypes.data_as(C.POINTER(C.c_float)) if want_logits else None
-        _lib.check(self._h, _lib.lib().nl_prefill(self._h, stream, arr, len(tokens), int(pos0), out))
+        self._check(self._L.nl_prefill(self._h, stream, arr, len(tokens), int(pos0), out))
 
     def forward_batch(self, streams: List[int], tokens: List[int], pos: List[int], want_logits: bool = False):
         n = len(streams)
         ia = lambda v: (C.c_int * n)(*[int(x) for x in v])
         ids = (C.c_int * n)()
         lg = np.zeros((n, self.config.vocab_size), dtype=np.float32) if want_logits else None
-        _lib.check(self._h, _lib.lib().nl_forward_batch(
+        self._check(self._L.nl_forward_batch(
             self._h, ia(streams), ia(tokens), ia(pos), n,
             lg.ctypes.data_as(C.POINTER(C.c_float)) if want_logits else None, ids))
         return [int(ids[i]) for i in range(n)], lg
+
+    def step(self, entries):
+        """One batch of token runs, one per stream: entries = [(stream, tokens, first position, wanted places)], results = the
+        logits at every entry's wanted places, [wanted, vocab] per entry.  (Families without a ragged step of their own: a run is
+        cut behind each wanted place.)"""
+        out = []
+        for stream, tokens, pos0, want in entries:
+            rows, at = np.zeros((len(want), self.config.vocab_size), np.float32), 0
+            for i, w in enumerate(want):
+                self.prefill(tokens[at:w + 1], pos0 + at, stream)
+                rows[i], at = self.state.logits, w + 1
+            if at < len(tokens):
+                self.prefill(tokens[at:], pos0 + at, stream, want_logits=False)
+            out.append(rows)
+        return out
+
+    # --- Reset go/model.go:623 ---
+    def reset(self, stream: int = 0) -> None:
+        self._check(self._L.nl_reset(self._h, stream))
+        self.state.pos = 0
+
+    # --- measurement / introspection ---
+    def synchronize(self):
+        self._check(self._L.nl_synchronize(self._h))
+
+    def timer_start(self):
+        self._check(self._L.nl_timer_start(self._h))
+
+    def timer_stop(self) -> float:
+        ms = C.c_float(0)
+        self._check(self._L.nl_timer_stop(self._h, C.byref(ms)))
+        return ms.value
+
+    def memory_usage(self):
+        w, kv, st = C.c_uint64(0), C.c_uint64(0), C.c_uint64(0)
+        self._check(self._L.nl_memory_usage(self._h, C.byref(w), C.byref(kv), C.byref(st)))
+        return {"weights": w.value, "kv_cache": kv.value, "state": st.value}
+
+    def last_error(self) -> str:
+        """nl_last_error: the message of the last failed call -- or the one-time note of a call that succeeded after
+        retiring the fused launch plan (a cluster exchange timed out and the step was redone on the general plan)."""
+        return (self._L.nl_last_error(self._h) or b"").decode()
+
+    def debug_read(self, which: str, n: int, stream: int = 0) -> np.ndarray:
+        out = np.zeros(n, dtype=np.float32)
+        got = self._L.nl_debug_read(self._h, which.encode(), stream, out.ctypes.data_as(C.POINTER(C.c_float)), n)
+        if got < 0:
+            self._check(int(got))
+        return out[:got]
+
+    def close(self):
+        if self._h:
+            self._L.nl_destroy(self._h)
+            self._h = None
+
+    def __del__(self):
+        try:
+            self.close()
+        except Exception:
+            pass
+
+
+class LlamaModel(HipModel):
+    """The quantised Llama family (GGUF), libnanollama_hip.so."""
+
+    def __init__(self, config: LlamaConfig, handle, max_streams: int):
+        super().__init__(config, handle, max_streams, _lib.lib())
 
     def set_gamma(self, indices, values) -> None:
         """model.Gamma = gamma (go/main.go:79): indices int32 [n], values [n, dim] float32 or float16."""
@@ -122,80 +195,34 @@ class LlamaModel:
             vals = vals.astype(np.float32)
         if idx.size and (vals.ndim != 2 or vals.shape != (idx.size, self.config.embed_dim)):
             raise ValueError(f"gamma embed_dim {vals.shape} != model dim {self.config.embed_dim}")  # go/main.go:75-77
-        _lib.check(self._h, _lib.lib().nl_set_gamma(self._h, idx.ctypes.data_as(C.POINTER(C.c_int32)), int(idx.size),
+        self._check(self._L.nl_set_gamma(self._h, idx.ctypes.data_as(C.POINTER(C.c_int32)), int(idx.size),
                                                     vals.ctypes.data, int(vals.dtype == np.float16)))
         self.gamma = (idx, vals) if idx.size else None
 
-    # --- Reset go/model.go:623 ---
-    def reset(self, stream: int = 0) -> None:
-        _lib.check(self._h, _lib.lib().nl_reset(self._h, stream))
-        self.state.pos = 0
-
-    # --- measurement / introspection ---
-    def synchronize(self):
-        _lib.check(self._h, _lib.lib().nl_synchronize(self._h))
-
-    def timer_start(self):
-        _lib.check(self._h, _lib.lib().nl_timer_start(self._h))
-
-    def timer_stop(self) -> float:
-        ms = C.c_float(0)
-        _lib.check(self._h, _lib.lib().nl_timer_stop(self._h, C.byref(ms)))
-        return ms.value
-
     def profile_forward(self, token: int, pos: int, iters: int = 10, stream: int = 0):
-        L = _lib.lib()
         ms = (C.c_float * _lib.NL_NUM_KINDS)()
         calls = (C.c_int * _lib.NL_NUM_KINDS)()
-        _lib.check(self._h, L.nl_profile_forward(self._h, stream, token, pos, iters, ms, calls))
-        return {L.nl_kernel_kind_name(k).decode(): (ms[k], calls[k]) for k in range(_lib.NL_NUM_KINDS)}
-
-    def memory_usage(self):
-        w, kv, st = C.c_uint64(0), C.c_uint64(0), C.c_uint64(0)
-        _lib.check(self._h, _lib.lib().nl_memory_usage(self._h, C.byref(w), C.byref(kv), C.byref(st)))
-        return {"weights": w.value, "kv_cache": kv.value, "state": st.value}
+        self._check(self._L.nl_profile_forward(self._h, stream, token, pos, iters, ms, calls))
+        return {self._L.nl_kernel_kind_name(k).decode(): (ms[k], calls[k]) for k in range(_lib.NL_NUM_KINDS)}
 
     def p2p_info(self):
         """Tensor-parallel transport of this handle: push all-reduce set up? receive area uncached?"""
         on, unc = C.c_int(0), C.c_int(0)
-        _lib.check(self._h, _lib.lib().nl_p2p_info(self._h, C.byref(on), C.byref(unc)))
+        self._check(self._L.nl_p2p_info(self._h, C.byref(on), C.byref(unc)))
         return {"push_allreduce": bool(on.value), "uncached_receive_area": bool(unc.value)}
 
     def plan_info(self):
         """nl_plan_info: which launch plans the handle holds (fused mode, its position limit, launches per token)."""
         v = [C.c_int(0) for _ in range(4)]
-        _lib.check(self._h, _lib.lib().nl_plan_info(self._h, *[C.byref(x) for x in v]))
+        self._check(self._L.nl_plan_info(self._h, *[C.byref(x) for x in v]))
         return {"fused_mode": v[0].value, "fused_max_pos": v[1].value, "launches_fused": v[2].value, "launches_general": v[3].value}
 
     def persist_info(self):
         """nl_persist_info: is the one-launch-per-chunk persistent decode (nl_persist.h) serving greedy chains of this handle."""
         ready, max_pos = C.c_int(0), C.c_int(0)
         launches, tokens = C.c_longlong(0), C.c_longlong(0)
-        _lib.check(self._h, _lib.lib().nl_persist_info(self._h, C.byref(ready), C.byref(max_pos), C.byref(launches), C.byref(tokens)))
+        self._check(self._L.nl_persist_info(self._h, C.byref(ready), C.byref(max_pos), C.byref(launches), C.byref(tokens)))
         return {"ready": bool(ready.value), "max_pos": max_pos.value, "launches": launches.value, "tokens": tokens.value}
-
-    def last_error(self) -> str:
-        """nl_last_error: the message of the last failed call -- or the one-time note of a call that succeeded after
-        retiring the fused launch plan (a cluster exchange timed out and the step was redone on the general plan)."""
-        return (_lib.lib().nl_last_error(self._h) or b"").decode()
-
-    def debug_read(self, which: str, n: int, stream: int = 0) -> np.ndarray:
-        out = np.zeros(n, dtype=np.float32)
-        got = _lib.lib().nl_debug_read(self._h, which.encode(), stream, out.ctypes.data_as(C.POINTER(C.c_float)), n)
-        if got < 0:
-            _lib.check(self._h, int(got))
-        return out[:got]
-
-    def close(self):
-        if self._h:
-            _lib.lib().nl_destroy(self._h)
-            self._h = None
-
-    def __del__(self):
-        try:
-            self.close()
-        except Exception:
-            pass
 
 
 def load_llama_model(gguf: GGUFFile, device: int = 0, max_streams: int = 1, tp_rank: int = 0, tp_size: int = 1,
