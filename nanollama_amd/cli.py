@@ -3,6 +3,7 @@
     python -m nanollama_amd --model m.gguf --prompt "Hello"            (one shot)
     python -m nanollama_amd --model m.gguf --interactive               (REPL, /quit /exit /info)
     python -m nanollama_amd --model m.gguf --serve --port 8080         (HTTP: GET /, POST /chat, GET /health)
+    python -m nanollama_amd --model folder --prompt "12 7 345"         (config.json + model.safetensors: prompts are token ids)
 """
 from __future__ import annotations
 
@@ -14,12 +15,13 @@ from .engine import GenParams
 from .engine_text import TextEngine
 from .gguf import GGUFError, load_gguf
 from .model import load_llama_model
-from .tokenizer import Tokenizer
+from .registry import is_model_folder, load_model, read_spec
+from .tokenizer import IdTokenizer, Tokenizer
 
 
 def build_parser() -> argparse.ArgumentParser:
     ap = argparse.ArgumentParser(prog="nanollama", description="nanollama inference on MI355X (GGUF in, text out)")
-    ap.add_argument("--model", default="", help="Path to GGUF model file (required)")
+    ap.add_argument("--model", default="", help="Path to a GGUF model file or a model folder (required)")
     ap.add_argument("--gamma", default="", help="Path to gamma NPZ file (optional, personality)")
     ap.add_argument("--prompt", default="", help="Prompt text (if empty, reads from stdin)")
     ap.add_argument("--max-tokens", type=int, default=256, help="Maximum tokens to generate")
@@ -36,12 +38,16 @@ def build_parser() -> argparse.ArgumentParser:
     ap.add_argument("--gpus", type=int, default=1,
                     help="shard the model tensor-parallel over this many GPUs of the node (2, 4 or 8: devices --device .. --device + N - 1; "
                          "the 7.9B tier's configuration).  One process, one engine: --serve and --interactive work unchanged")
+    ap.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16", help="arithmetic of a model folder's products (GGUF files: fixed by the format)")
+    ap.add_argument("--seq-len", type=int, default=0, help="model folders: positions to allocate for (0: the default)")
     ap.add_argument("--seed", type=int, default=None, help="sampling seed (default: entropy, like the reference)")
     return ap
 
 
 def estimate_params(cfg) -> int:
-    """estimateParams go/main.go:411-425"""
+    """estimateParams go/main.go:411-425 (model folders: counted)"""
+    if hasattr(cfg, "num_params"):
+        return cfg.num_params
     embed = cfg.vocab_size * cfg.embed_dim
     attn = cfg.embed_dim * (cfg.num_heads * cfg.head_dim) + 2 * cfg.embed_dim * (cfg.num_kv_heads * cfg.head_dim) + \
         cfg.embed_dim * cfg.embed_dim
@@ -55,8 +61,25 @@ def list_tensors(g) -> None:
         print("  %-50s  type=%d  dims=[%s]  %.2f MB" % (name, info.type, dims, info.nbytes() / 1024 / 1024))
 
 
+def list_folder_tensors(path: str) -> None:
+    _, w = read_spec(path)
+    for name in w.names():
+        print("  %-50s  dims=[%s]  %.2f MB" % (name, ", ".join(str(d) for d in w.shape(name)), w.nbytes(name) / 1024 / 1024))
+
+
+def load_folder_engine(args) -> TextEngine:
+    if args.gpus > 1 or args.gamma:
+        raise RuntimeError("--gpus and --gamma are for GGUF models")
+    model = load_model(args.model, device=args.device, dtype=args.dtype, seq_len=args.seq_len, verbose=True)
+    c = model.config
+    print("[nanollama] ready — %s, %dM params, %d layers, %d dim" % (c.architecture, estimate_params(c) // 1_000_000, c.num_layers, c.embed_dim))
+    return TextEngine(model, IdTokenizer(c.vocab_size), rep_penalty=args.rep_penalty, rep_window=args.rep_window, seed=args.seed)
+
+
 def load_engine(args) -> TextEngine:
     print(f"[nanollama] loading {args.model}")
+    if is_model_folder(args.model):
+        return load_folder_engine(args)
     g = load_gguf(args.model, verbose=True)
     if args.gpus > 1:
         if args.gpus not in (2, 4, 8):
@@ -105,7 +128,10 @@ def run_repl(eng: TextEngine, params: GenParams) -> None:
             print(f"Gamma: {eng.model.gamma is not None}")
             print(f"Flags: qk_norm={c.qk_norm} rope_conjugate={c.rope_conjugate}")
             continue
-        eng.generate(text, params, stream=sys.stdout)
+        try:
+            eng.generate(text, params, stream=sys.stdout)
+        except ValueError as exc:
+            print(f"error: {exc}")
         print()
 
 
@@ -117,10 +143,13 @@ def main(argv=None) -> int:
         return 1
     try:
         if args.list_tensors:
-            list_tensors(load_gguf(args.model, verbose=True))
+            if is_model_folder(args.model):
+                list_folder_tensors(args.model)
+            else:
+                list_tensors(load_gguf(args.model, verbose=True))
             return 0
         eng = load_engine(args)
-    except (GGUFError, OSError, RuntimeError, ImportError) as exc:
+    except (GGUFError, OSError, RuntimeError, ImportError, ValueError, KeyError) as exc:
         print(f"error: {exc}", file=sys.stderr)
         return 1
     params = GenParams(max_tokens=args.max_tokens, temperature=args.temp, top_p=args.top_p, top_k=args.top_k)
@@ -130,7 +159,11 @@ def main(argv=None) -> int:
     elif args.interactive:
         run_repl(eng, params)
     elif args.prompt:
-        print(eng.generate(args.prompt, params, stream=sys.stdout))
+        try:
+            print(eng.generate(args.prompt, params, stream=sys.stdout))
+        except ValueError as exc:                   # a prompt the model's tokenizer cannot take
+            print(f"error: {exc}", file=sys.stderr)
+            return 1
     else:
         print("> ", end="", flush=True)
         for line in sys.stdin:

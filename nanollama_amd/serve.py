@@ -50,8 +50,11 @@ def handle_chat(engine, defaults: GenParams, lock: threading.Lock, body: bytes):
         params = replace(params, temperature=float(req["temperature"]))
     if isinstance(req.get("top_k"), (int, float)) and req["top_k"] > 0:
         params = replace(params, top_k=int(req["top_k"]))
-    with lock:
-        result = engine.generate_quiet(prompt, params)
+    try:
+        with lock:
+            result = engine.generate_quiet(prompt, params)
+    except ValueError as exc:                # a prompt the model's tokenizer cannot take
+        return 400, "bad request: " + str(exc)
     return 200, {"response": result}
 
 

@@ -208,3 +208,26 @@ class Tokenizer:
             if v in self.token_to_id:
                 return self.token_to_id[v]
         return -1
+
+
+class IdTokenizer:
+    """Text <-> ids for models that come without a vocabulary: a prompt is whitespace-separated token ids."""
+
+    def __init__(self, vocab_size: int):
+        self.vocab_size = vocab_size
+        self.bos_id = self.eos_id = -1
+
+    def encode(self, text: str, add_bos: bool = True) -> List[int]:
+        ids = [int(t) for t in text.split()]        # ValueError for anything but integers
+        bad = [t for t in ids if not 0 <= t < self.vocab_size]
+        if bad:
+            raise ValueError(f"token id {bad[0]} outside [0, {self.vocab_size})")
+        if not ids:
+            raise ValueError("empty prompt")
+        return ids
+
+    def decode_token_bytes(self, tid: int) -> bytes:
+        return b"%d " % tid
+
+    def decode(self, ids: List[int]) -> str:
+        return "".join("%d " % t for t in ids)
