@@ -660,6 +660,102 @@ def shard_probe(model, rdv, ns=(2, 4, 8), seam_us=2.0, steps=96, warmup=16, base
     return out
 
 
+# ------------------------------------------------------------------ layer-stack models (--stack) ---
+
+def stack_sizes():
+    """name -> (Llama shape, Ganidra configuration) of equal width, depth, feed-forward and vocabulary.  Every fourth Ganidra layer is
+    a parallel one (softmax attention over a 1024-token window beside linear attention), the others are linear attention."""
+    from nanollama_amd import synth
+    from nanollama_amd.synth_stack import ganidra_config, ganidra_layer
+    out = {}
+    for name, L, D, V in (("mini", 20, 768, 32000), ("goldie", 28, 1536, 48000), ("wide", 4, 4096, 32000)):
+        shape = synth.ModelShape("stackbench_" + name, L, D, D // 64, D // 256, V)
+        lin = lambda h: dict(heads=h, dim=64, vdim=128, tau=16.0)
+        par = ganidra_layer("parallel", shape.ffn, left=dict(heads=D // 128, kv_heads=max(1, D // 512), dim=64, vdim=64, scale=0.125, mask={"size": 1024}),
+                            left_scale=0.7, right=lin(D // 256), right_scale=0.7)
+        gla = ganidra_layer("gla", shape.ffn, **lin(D // 128))
+        out[name] = (shape, ganidra_config(V, D, [par if i % 4 == 3 else gla for i in range(L)]))
+    return out
+
+
+def time_model(dev, vocab, streams, prompt_len=2047, pos=512, steps=128, batch_steps=32):
+    """Prompt, single-stream greedy decode and a batch of decode streams of one loaded model (host wall clock, best of three)."""
+    import numpy as np
+    from nanollama_amd import synth
+    toks = synth.prompt_ids(prompt_len, vocab)
+
+    def best(f, reps=3):
+        t = []
+        for _ in range(reps):
+            dev.synchronize()
+            t0 = time.perf_counter()
+            f()
+            dev.synchronize()
+            t.append(time.perf_counter() - t0)
+        return min(t)
+
+    def prompt():
+        dev.reset()
+        dev.prefill(toks)
+    prompt()
+    out = {"prompt_tokens": prompt_len, "prefill_ms": round(best(prompt) * 1e3, 3)}
+    out["prefill_tokens_per_s"] = round(prompt_len / out["prefill_ms"] * 1e3)
+
+    def chain():
+        dev.reset()
+        dev.prefill(toks[:pos], want_logits=False)
+        dev.synchronize()
+        t0 = time.perf_counter()
+        for i in range(0, steps, 64):
+            dev.decode_greedy(5, pos + i, 64)
+        return time.perf_counter() - t0
+    chain()
+    dt = min(chain() for _ in range(3))
+    out.update(decode_position=pos, decode_ms=round(dt / steps * 1e3, 4), decode_tokens_per_s=round(steps / dt, 1))
+    ids = list(range(streams))
+    for s in ids:
+        dev.reset(s)
+        dev.prefill(toks[:64], 0, s, want_logits=False)
+    at = [64]
+
+    def batch(n):
+        for _ in range(n):
+            dev.forward_batch(ids, [7 + s for s in ids], [at[0]] * streams)
+            at[0] += 1
+    batch(4)
+    dt = best(lambda: batch(batch_steps)) / batch_steps
+    out.update(batch_streams=streams, batch_ms_per_step=round(dt * 1e3, 4), batch_tokens_per_s=round(streams / dt))
+    return out
+
+
+def stack_bench(names, only=None):
+    """Ganidra (bfloat16) beside the quantised family's F16 files of equal size; random weights."""
+    from nanollama_amd import _lib, gguf, model, synth_stack
+    from nanollama_amd.designs import DESIGNS
+    from nanollama_amd.stack import load_stack_model
+    res = {}
+    for name in names:
+        shape, cfg = stack_sizes()[name]
+        r = {}
+        if only != "llama":
+            w = synth_stack.ganidra_weights(cfg, 1, fast=True)
+            spec = DESIGNS["Ganidra"](cfg, lambda n: w[n].shape)
+            dev = load_stack_model(spec, lambda n: ("BF16", w[n]), max_streams=64, seq_len=4096)
+            r["ganidra_bf16"] = dict(time_model(dev, shape.vocab, 64), params_millions=dev.config.num_params // 1000000)
+            dev.close()
+            del w
+        if only != "ganidra":
+            g = gguf.load_gguf(ensure_gguf(shape, "f16", "float"))
+            dev = model.load_llama_model(g, max_streams=64)
+            r["llama_f16"] = dict(time_model(dev, shape.vocab, 64), params_millions=(shape.matrix_params() + shape.vocab * shape.dim) // 1000000)
+            dev.close()
+        res[name] = r
+        print(f"[bench] {name}: {json.dumps(r)}", file=sys.stderr, flush=True)
+    return {"metric": "layer-stack model (Ganidra) and F16 Llama of equal size: prefill / decode / 64-stream decode", "unit": "tokens/s",
+            "value": res[names[-1]].get("ganidra_bf16", {}).get("decode_tokens_per_s"), "n_gpus": 1, "higher_is_better": True, "vs_baseline": None,
+            "dtype": "bf16", "data": "synthetic (random weights)", "sizes": res, "lib": _lib.source_sha(_lib.source_files("stack"))}
+
+
 def workload_text(shape, tier, wtype, r, steps):
     """What the timed region ran: `steps` chained greedy decode steps as segments that each restart behind the prompt."""
     seg = r["segment"]
@@ -697,7 +793,13 @@ def main():
     ap.add_argument("--no-shard-probe", action="store_true", help="N = 1: skip the tensor-parallel shard-only probe of big")
     ap.add_argument("--rccl-worker", default=None, help=argparse.SUPPRESS)
     ap.add_argument("--profile-pos", type=int, default=None, help="position of the per-launch profile (default: the mean timed position)")
+    ap.add_argument("--stack", nargs="?", const="mini,goldie,wide", default=None, metavar="SIZES",
+                    help="one GPU: time the layer-stack design beside an F16 Llama of equal size and print that line only")
+    ap.add_argument("--stack-only", choices=("ganidra", "llama"), default=None, help="with --stack: one of the two models")
     args = ap.parse_args()
+    if args.stack:
+        print(json.dumps(stack_bench(args.stack.split(","), args.stack_only)))
+        return
     n = args.gpus
     if n < 1:
         raise SystemExit("--gpus must be >= 1")

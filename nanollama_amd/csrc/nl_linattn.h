@@ -39,7 +39,7 @@ struct GlaParams {
     int ldp, off_q, off_k, off_v, off_g, off_a1;
     int heads, dk, dv, rank;
     int dkp, dvp;              // dk, dv rounded up to 16: the state's leading dimensions
-    const float *a2, *a2b, *norm;   // [heads * dk][rank], [heads * dk], [dv]
+    const float *a2, *a2b, *norm;   // [rank][heads * dk], [heads * dk], [dv]
     float tau, eps, qscale, oscale;
     float *state;              // this layer run, stream 0: [heads][dkp][dvp]
     long long state_stride;    // floats per stream
@@ -54,60 +54,114 @@ struct GlaParams {
     const int *runs;           // gla_scan_kernel: first segment of every run with more than one segment
 };
 
-__device__ __forceinline__ float gla_log_alpha(float z, float tau) { return (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) / tau; }
+// log sigmoid(z) / tau = (min(z, 0) - log1p(e)) / tau, e = exp(-|z|) in (0, 1]: log1p by the area-tangent series
+// log(1 + e) = 2 (s + s^3 / 3 + s^5 / 5 + ...), s = e / (2 + e) <= 1 / 3, cut behind s^17 (relative error below 2e-9)
+__device__ __forceinline__ float gla_log_alpha(float z, float inv_tau) {
+    const float e = exp_f32(-fminf(fabsf(z), 1e4f)), s = e * rcp_f32(2.f + e), w = s * s;
+    float p = 1.f / 17.f;
+    p = fmaf(p, w, 1.f / 15.f);
+    p = fmaf(p, w, 1.f / 13.f);
+    p = fmaf(p, w, 1.f / 11.f);
+    p = fmaf(p, w, 1.f / 9.f);
+    p = fmaf(p, w, 1.f / 7.f);
+    p = fmaf(p, w, 1.f / 5.f);
+    p = fmaf(p, w, 1.f / 3.f);
+    return (fminf(z, 0.f) - 2.f * fmaf(s * w, p, s)) * inv_tau;
+}
 
 // grid (sub-chunks, channels / 256)
 __global__ void __launch_bounds__(256) gla_decay_kernel(GlaParams P) {
     extern __shared__ __align__(16) char lds[];
-    float *a1 = reinterpret_cast<float *>(lds);                  // [16][rank]
+    float *a1 = reinterpret_cast<float *>(lds);                  // [rank][16]
     const GlaSub sc = P.subs[blockIdx.x];
-    for (int i = threadIdx.x; i < sc.len * P.rank; i += 256) {
-        const int t = i / P.rank;
-        a1[i] = P.proj[(long long)(sc.tok0 + t) * P.ldp + P.off_a1 + (i - t * P.rank)];
+    for (int i = threadIdx.x; i < LA_SUB * P.rank; i += 256) {
+        const int t = i / P.rank, r = i - t * P.rank;
+        a1[r * LA_SUB + t] = t < sc.len ? P.proj[(long long)(sc.tok0 + t) * P.ldp + P.off_a1 + r] : 0.f;
     }
-    __syncthreads();
-    const int c = blockIdx.y * 256 + threadIdx.x, C = P.heads * P.dk;
-    if (c >= C) return;
-    const float *w = P.a2 + (long long)c * P.rank;
-    float z[LA_SUB];
-#pragma unroll
-    for (int t = 0; t < LA_SUB; t++) z[t] = 0.f;
-    for (int r = 0; r < P.rank; r++) {
-        const float wr = w[r];
-#pragma unroll
-        for (int t = 0; t < LA_SUB; t++)
-            if (t < sc.len) z[t] = fmaf(wr, a1[t * P.rank + r], z[t]);
-    }
-    float l = 0.f;
+    const int C = P.heads * P.dk, c = min((int)(blockIdx.y * 256 + threadIdx.x), C - 1);
     const float b = P.a2b[c];
+    f32x4 z[LA_SUB / 4];
 #pragma unroll
-    for (int t = 0; t < LA_SUB; t++)
-        if (t < sc.len) {
-            l += gla_log_alpha(z[t] + b, P.tau);
-            P.ldec[(long long)(sc.tok0 + t) * C + c] = l;
+    for (int q = 0; q < LA_SUB / 4; q++) z[q] = f32x4{b, b, b, b};
+    __syncthreads();
+#pragma unroll 8
+    for (int r = 0; r < P.rank; r++) {
+        const float wr = P.a2[(long long)r * C + c];
+#pragma unroll
+        for (int q = 0; q < LA_SUB / 4; q++) {
+            const f32x4 x = *reinterpret_cast<const f32x4 *>(a1 + r * LA_SUB + q * 4);
+#pragma unroll
+            for (int i = 0; i < 4; i++) z[q][i] = fmaf(wr, x[i], z[q][i]);
         }
+    }
+    const float it = 1.f / P.tau;
+    float l = 0.f;
+#pragma unroll
+    for (int t = 0; t < LA_SUB; t++) {
+        l += gla_log_alpha(z[t >> 2][t & 3], it);
+        if (t < sc.len && (int)(blockIdx.y * 256 + threadIdx.x) < C) P.ldec[(long long)(sc.tok0 + t) * C + c] = l;
+    }
 }
 
-// grid (segments, heads), dvp / 16 wavefronts; wavefront w owns value columns 16 w .. 16 w + 15
-template <typename T, int DKT, bool OUT>
-__global__ void __launch_bounds__(1024) gla_seg_kernel(GlaParams P) {
+// grid (segments, heads), max(dvp, dkp) / 16 wavefronts; wavefront w < dvp / 16 owns value columns 16 w .. 16 w + 15, all of them load.
+// The next sub-chunk's operands are requested before the current one is multiplied.
+// NE: operand elements per thread, at least 16 dkp / threads (at most 4); WV: most wavefronts of a launch
+template <typename T, int DKT, int NE, int WV, bool OUT>
+__global__ void __launch_bounds__(WV * 64) gla_seg_kernel(GlaParams P) {
     extern __shared__ __align__(16) char lds[];
     const GlaSeg sg = P.segs[blockIdx.x];
     if (!OUT && (sg.nseg == 1 || sg.index + 1 == sg.nseg)) return;     // nobody starts from the state behind the last segment
     const int h = blockIdx.y, tid = threadIdx.x, nthr = blockDim.x, lane = tid & 63, w = tid >> 6, nw = nthr >> 6, g = lane >> 4, c = lane & 15;
     const int dk = P.dk, dkp = P.dkp, nkt = dkp >> 4, ld = dkp + 4, C = P.heads * dk, dvc = w * 16 + c;
+    const int nv = P.dvp >> 4;
+    const bool owner = w < nv, value = dvc < P.dv;
     float *qd = reinterpret_cast<float *>(lds);          // [16][ld]  q e^l
     float *ki = qd + 16 * ld;                            // [16][ld]  k e^-l
     float *ke = ki + 16 * ld;                            // [16][ld]  k e^{l_end - l}
-    float *tot = ke + 16 * ld;                           // [dkp]     l_end
-    float *A = tot + dkp;                                // [16][20]
-    float *part = A + 16 * 20;                           // [nw][256] partial A, then [nw][16] sums of squares
+    float *etot = ke + 16 * ld;                          // [dkp]     e^{l_end}
+    float *A = etot + dkp;                                // [16][20]
+    float *ssq = A + 16 * 20;                            // [nw][16] sums of squares
+    int *flag = reinterpret_cast<int *>(ssq + nw * 16);  // [16] wavefront saw a decay beyond the factored range
+    float *part = ssq + nw * 16 + 16;                    // [nw][256] partial A
     f32x4 S[DKT];
     const long long shead = (long long)dkp * P.dvp;
     float *stream_state = P.state + sg.stream * P.state_stride + h * shead;
     float *seg_state = P.inc + ((long long)blockIdx.x * P.heads + h) * shead;
+    const int nsub = (sg.len + LA_SUB - 1) / LA_SUB;
+    float rq[NE], rk[NE], rl[NE], re[NE], rv[4], rg[4];
+    int et[NE], ed[NE];                                  // this thread's elements: token of the sub-chunk (16: none), channel
+#pragma unroll
+    for (int e = 0; e < NE; e++) {
+        const int i = tid + e * nthr;
+        et[e] = min(i / dkp, LA_SUB);
+        ed[e] = i - i / dkp * dkp;
+    }
+    const char *proj = reinterpret_cast<const char *>(P.proj + (long long)sg.tok0 * P.ldp), *ldec = reinterpret_cast<const char *>(P.ldec + (long long)sg.tok0 * C + h * dk);
+    auto fetch = [&](int sub) {
+        const int u0 = sub * LA_SUB, len = min(LA_SUB, sg.len - u0);
+#pragma unroll
+        for (int e = 0; e < NE; e++) {
+            rq[e] = rk[e] = rl[e] = re[e] = 0.f;
+            if (et[e] < LA_SUB && ed[e] < dk) {
+                re[e] = ld_off<float>(ldec, (unsigned)((u0 + len - 1) * C + ed[e]) * 4u);
+                if (et[e] < len) {
+                    const unsigned at = (unsigned)((u0 + et[e]) * P.ldp + h * dk + ed[e]);
+                    rk[e] = ld_off<float>(proj, (at + P.off_k) * 4u);
+                    rl[e] = ld_off<float>(ldec, (unsigned)((u0 + et[e]) * C + ed[e]) * 4u);
+                    if (OUT) rq[e] = ld_off<float>(proj, (at + P.off_q) * 4u);
+                }
+            }
+        }
+        // value columns in B-operand order: step s holds token 4 s + g; the gates in accumulator order: token 4 g + i
+#pragma unroll
+        for (int s = 0; s < 4; s++) {
+            rv[s] = owner && value && 4 * s + g < len ? ld_off<float>(proj, (unsigned)((u0 + 4 * s + g) * P.ldp + P.off_v + h * P.dv + dvc) * 4u) : 0.f;
+            if (OUT) rg[s] = owner && value && 4 * g + s < len ? ld_off<float>(proj, (unsigned)((u0 + 4 * g + s) * P.ldp + P.off_g + h * P.dv + dvc) * 4u) : 0.f;
+        }
+    };
+    fetch(0);
     {
-        const float *from = !OUT ? nullptr : sg.nseg > 1 ? seg_state : sg.pos0 == 0 ? nullptr : stream_state;
+        const float *from = !OUT || !owner ? nullptr : sg.nseg > 1 ? seg_state : sg.pos0 == 0 ? nullptr : stream_state;
 #pragma unroll
         for (int dt = 0; dt < DKT; dt++) {
             S[dt] = f32x4{};
@@ -116,106 +170,123 @@ __global__ void __launch_bounds__(1024) gla_seg_kernel(GlaParams P) {
                 for (int i = 0; i < 4; i++) S[dt][i] = from[(long long)(dt * 16 + 4 * g + i) * P.dvp + dvc];
         }
     }
-    const int nsub = (sg.len + LA_SUB - 1) / LA_SUB;
+    const float inv_dv = 1.f / (float)P.dv;
+    const int ycol = (int)op_index(0, P.y_k0 + h * P.dv + dvc, P.y_nks);
+    const float nrm = OUT && value ? P.norm[dvc] * P.oscale : 0.f;
     for (int sub = 0; sub < nsub; sub++) {
         const int t0 = sg.tok0 + sub * LA_SUB, len = min(LA_SUB, sg.len - sub * LA_SUB);
         // operands of the sub-chunk; tokens beyond its length and channels beyond dk are zero
         bool strong = false;
-        for (int i = tid; i < LA_SUB * dkp; i += nthr) {
-            const int t = i / dkp, d = i - t * dkp;
-            float q = 0.f, k = 0.f, l = 0.f, le = 0.f;
-            if (d < dk) le = P.ldec[(long long)(t0 + len - 1) * C + h * dk + d];
-            if (t < len && d < dk) {
-                const long long at = (long long)(t0 + t) * P.ldp + h * dk + d;
-                k = P.proj[at + P.off_k];
-                l = P.ldec[(long long)(t0 + t) * C + h * dk + d];
-                if (OUT) q = P.proj[at + P.off_q] * P.qscale;
-            }
-            ke[t * ld + d] = k * expf(le - l);
-            if (OUT) {
-                strong |= le < -LA_FACTOR_MAX;
-                qd[t * ld + d] = q * expf(l);
-                ki[t * ld + d] = k * expf(fminf(-l, LA_FACTOR_MAX));
-            }
-            if (t == 0) tot[d] = le;
-        }
-        // this wavefront's value columns, in B-operand order: step s holds token 4 s + g
-        float v[4];
 #pragma unroll
-        for (int s = 0; s < 4; s++)
-            v[s] = 4 * s + g < len && dvc < P.dv ? P.proj[(long long)(t0 + 4 * s + g) * P.ldp + P.off_v + h * P.dv + dvc] : 0.f;
+        for (int e = 0; e < NE; e++) {
+            const int t = et[e], d = ed[e];
+            if (t < LA_SUB) {
+                ke[t * ld + d] = rk[e] * exp_f32(re[e] - rl[e]);
+                if (OUT) {
+                    strong |= re[e] < -LA_FACTOR_MAX;
+                    qd[t * ld + d] = rq[e] * P.qscale * exp_f32(rl[e]);
+                    ki[t * ld + d] = rk[e] * exp_f32(fminf(-rl[e], LA_FACTOR_MAX));
+                }
+                if (t == 0) etot[d] = exp_f32(re[e]);
+            }
+        }
+        float v[4], gz[4];
+#pragma unroll
+        for (int s = 0; s < 4; s++) { v[s] = rv[s]; gz[s] = rg[s]; }
         if (OUT) {
-            const bool slow = __syncthreads_or(strong);
+            const bool any = __any(strong);
+            if (lane == 0) flag[w] = any;
+        }
+        lds_barrier();
+        if (sub + 1 < nsub) fetch(sub + 1);
+        bool slow = false;
+        if (OUT)
+            for (int q = 0; q < nw; q++) slow |= flag[q] != 0;
+        f32x4 o = {};
+        if (OUT) {
             if (!slow) {
                 f32x4 a = {};
                 for (int ks = w; ks < dkp / 4; ks += nw)
                     a = __builtin_amdgcn_mfma_f32_16x16x4f32(qd[c * ld + 4 * ks + g], ki[c * ld + 4 * ks + g], a, 0, 0, 0);
 #pragma unroll
                 for (int i = 0; i < 4; i++) part[w * 256 + (4 * g + i) * 16 + c] = a[i];
-                __syncthreads();
             }
+            if (owner) {
+#pragma unroll
+                for (int dt = 0; dt < DKT; dt++)
+                    if (dt < nkt) {
+                        const f32x4 qv = *reinterpret_cast<const f32x4 *>(qd + c * ld + dt * 16 + 4 * g);
+#pragma unroll
+                        for (int i = 0; i < 4; i++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(qv[i], S[dt][i], o, 0, 0, 0);
+                    }
+            }
+        }
+        if (owner) {
+#pragma unroll
+            for (int dt = 0; dt < DKT; dt++)
+                if (dt < nkt) {
+                    const f32x4 tl = *reinterpret_cast<const f32x4 *>(etot + dt * 16 + 4 * g);
+#pragma unroll
+                    for (int i = 0; i < 4; i++) S[dt][i] *= tl[i];
+#pragma unroll
+                    for (int s = 0; s < 4; s++) S[dt] = __builtin_amdgcn_mfma_f32_16x16x4f32(ke[(4 * s + g) * ld + dt * 16 + c], v[s], S[dt], 0, 0, 0);
+                }
+        }
+        lds_barrier();
+        if (OUT) {
             for (int i = tid; i < 256; i += nthr) {
                 const int t = i >> 4, s = i & 15;
                 float a = 0.f;
                 if (s <= t && t < len) {
                     if (!slow) {
-                        for (int q = 0; q < nw; q++) a += part[q * 256 + i];
+                        const int np = min(nw, dkp / 4);
+                        for (int q0 = 0; q0 < np; q0 += 8) {
+                            float x[8];
+#pragma unroll
+                            for (int q = 0; q < 8; q++) x[q] = part[min(q0 + q, np - 1) * 256 + i];
+#pragma unroll
+                            for (int q = 0; q < 8; q++) a += q0 + q < np ? x[q] : 0.f;
+                        }
                     } else {
                         const float *qp = P.proj + (long long)(t0 + t) * P.ldp + P.off_q + h * dk, *kp = P.proj + (long long)(t0 + s) * P.ldp + P.off_k + h * dk;
                         const float *lt = P.ldec + (long long)(t0 + t) * C + h * dk, *ls = P.ldec + (long long)(t0 + s) * C + h * dk;
-                        for (int d = 0; d < dk; d++) a += qp[d] * P.qscale * kp[d] * expf(lt[d] - ls[d]);
+#pragma unroll 1
+                        for (int d = 0; d < dk; d++) a += qp[d] * P.qscale * kp[d] * exp_f32(lt[d] - ls[d]);
                     }
                 }
                 A[t * 20 + s] = a;
             }
-        }
-        __syncthreads();
-        f32x4 o = {};
-        if (OUT) {
-#pragma unroll
-            for (int dt = 0; dt < DKT; dt++)
-                if (dt < nkt) {
-                    const f32x4 qv = *reinterpret_cast<const f32x4 *>(qd + c * ld + dt * 16 + 4 * g);
-#pragma unroll
-                    for (int i = 0; i < 4; i++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(qv[i], S[dt][i], o, 0, 0, 0);
-                }
+            lds_barrier();
 #pragma unroll
             for (int s = 0; s < 4; s++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(A[c * 20 + 4 * s + g], v[s], o, 0, 0, 0);
-        }
-#pragma unroll
-        for (int dt = 0; dt < DKT; dt++)
-            if (dt < nkt) {
-                const f32x4 tl = *reinterpret_cast<const f32x4 *>(tot + dt * 16 + 4 * g);
-#pragma unroll
-                for (int i = 0; i < 4; i++) S[dt][i] *= expf(tl[i]);
-#pragma unroll
-                for (int s = 0; s < 4; s++) S[dt] = __builtin_amdgcn_mfma_f32_16x16x4f32(ke[(4 * s + g) * ld + dt * 16 + c], v[s], S[dt], 0, 0, 0);
-            }
-        if (OUT) {
             // norm over the head's value columns: sums of squares over 16 lanes, then over the wavefronts
-            float ss[4];
 #pragma unroll
             for (int i = 0; i < 4; i++) {
-                ss[i] = o[i] * o[i];
+                float ss = o[i] * o[i];
 #pragma unroll
-                for (int m = 1; m < 16; m <<= 1) ss[i] += __shfl_xor(ss[i], m);
-                if (c == 0) part[w * 16 + 4 * g + i] = ss[i];
+                for (int m = 1; m < 16; m <<= 1) ss += __shfl_xor(ss, m);
+                if (c == 0) ssq[w * 16 + 4 * g + i] = ss;
             }
-            __syncthreads();
+            lds_barrier();
             T *y = reinterpret_cast<T *>(P.y);
+            f32x4 s2 = {};
+            for (int q0 = 0; q0 < nv; q0 += 4) {
+                f32x4 x[4];
 #pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const int t = 4 * g + i;
-                if (t < len && dvc < P.dv) {
-                    float tot2 = 0.f;
-                    for (int q = 0; q < nw; q++) tot2 += part[q * 16 + t];
-                    const float gz = P.proj[(long long)(t0 + t) * P.ldp + P.off_g + h * P.dv + dvc];
-                    const float r = o[i] / sqrtf(tot2 / (float)P.dv + P.eps) * P.norm[dvc] * (gz * sigmoid_f32(gz)) * P.oscale;
-                    put(y + op_index(t0 + t, P.y_k0 + h * P.dv + dvc, P.y_nks), r);
-                }
+                for (int q = 0; q < 4; q++) x[q] = *reinterpret_cast<const f32x4 *>(ssq + min(q0 + q, nv - 1) * 16 + 4 * g);
+#pragma unroll
+                for (int q = 0; q < 4; q++)
+                    if (q0 + q < nv) s2 += x[q];
             }
+            if (owner && value)
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const int t = 4 * g + i;
+                    if (t < len) {
+                        put(y + (unsigned)(((t0 + t) >> 4) * P.y_nks * OPT + ((t0 + t) & 15) * 8 + ycol), o[i] * rsqrt_f32(s2[i] * inv_dv + P.eps) * nrm * (gz[i] * sigmoid_f32(gz[i])));
+                    }
+                }
         }
-        __syncthreads();
     }
     if (!OUT) {
         // the segment's total log decay (every channel by one thread, from the sub-chunks' ends)
@@ -226,7 +297,7 @@ __global__ void __launch_bounds__(1024) gla_seg_kernel(GlaParams P) {
             P.totlog[((long long)blockIdx.x * P.heads + h) * dkp + d] = a;
         }
     }
-    if (!OUT || sg.index + 1 == sg.nseg) {
+    if (owner && (!OUT || sg.index + 1 == sg.nseg)) {
         float *to = OUT ? stream_state : seg_state;
 #pragma unroll
         for (int dt = 0; dt < DKT; dt++)
@@ -261,7 +332,7 @@ __global__ void __launch_bounds__(256) gla_scan_kernel(GlaParams P) {
         for (int u = 0; u < U; u++)
             if (i0 + u < sg.nseg) {
                 at[(i0 + u) * astep] = S;
-                S = S * expf(dec[u]) + inc[u];           // (the last segment's increment was not computed and is not used)
+                S = S * exp_f32(dec[u]) + inc[u];           // (the last segment's increment was not computed and is not used)
             }
     }
 }
@@ -271,12 +342,22 @@ __host__ __device__ inline size_t gla_decode_lds(int dkp, int dvp, int rank) { r
 
 template <typename T>
 __device__ __forceinline__ void gla_decode_block(const GlaParams &P, int h, int n, int stream, int pos, char *lds) {
-    const int tid = threadIdx.x, dk = P.dk, dv = P.dv;
+    constexpr int U = 8, RU = 16;
+    const int tid = threadIdx.x, dk = P.dk, dv = P.dv, C = P.heads * dk;
     float *q = reinterpret_cast<float *>(lds), *k = q + P.dkp, *al = k + P.dkp, *v = al + P.dkp, *part = v + P.dvp, *red = part + 1024, *a1 = red + 8;
     const float *pr = P.proj + (long long)n * P.ldp;
     const int nc = P.dvp >> 2, rp = 256 / nc, c4 = tid % nc, r0 = tid / nc;
     f32x4 *S = reinterpret_cast<f32x4 *>(P.state + stream * P.state_stride + (long long)h * P.dkp * P.dvp) + c4;
-    constexpr int U = 8;
+    // everything that does not depend on this step's arithmetic is requested up front (head sizes are at most 256: one element per
+    // thread), what is needed first in front: loads return in order
+    const bool kc = tid < dk, vc = tid < dv;
+    const float rq = kc ? pr[P.off_q + h * dk + tid] : 0.f, rk = kc ? pr[P.off_k + h * dk + tid] : 0.f, rv = vc ? pr[P.off_v + h * dv + tid] : 0.f;
+    const float ra = tid < P.rank ? pr[P.off_a1 + tid] : 0.f;
+    const float *w2 = P.a2 + h * dk + min(tid, dk - 1);
+    float w[RU];
+#pragma unroll
+    for (int r = 0; r < RU; r++) w[r] = w2[(long long)min(r, P.rank - 1) * C];
+    const float bias = kc ? P.a2b[h * dk + tid] : 0.f, gz = vc ? pr[P.off_g + h * dv + tid] : 0.f, nrm = vc ? P.norm[tid] * P.oscale : 0.f;
     f32x4 s[U];
     auto load = [&](int d0) {
 #pragma unroll
@@ -286,20 +367,20 @@ __device__ __forceinline__ void gla_decode_block(const GlaParams &P, int h, int 
         }
     };
     load(r0);
-    for (int i = tid; i < P.rank; i += 256) a1[i] = pr[P.off_a1 + i];
-    for (int i = tid; i < P.dvp; i += 256) v[i] = i < dv ? pr[P.off_v + h * dv + i] : 0.f;
-    for (int i = tid; i < dk; i += 256) {
-        q[i] = pr[P.off_q + h * dk + i] * P.qscale;
-        k[i] = pr[P.off_k + h * dk + i];
+    if (tid < P.rank) a1[tid] = ra;
+    for (int i = tid + 256; i < P.rank; i += 256) a1[i] = pr[P.off_a1 + i];
+    if (kc) { q[tid] = rq * P.qscale; k[tid] = rk; }
+    if (tid < P.dvp) v[tid] = rv;
+    lds_barrier();
+    if (kc) {
+        float z = bias;
+#pragma unroll
+        for (int r = 0; r < RU; r++)
+            if (r < P.rank) z = fmaf(w[r], a1[r], z);
+        for (int r = RU; r < P.rank; r++) z = fmaf(w2[(long long)r * C], a1[r], z);
+        al[tid] = exp_f32(gla_log_alpha(z, 1.f / P.tau));
     }
-    __syncthreads();
-    for (int i = tid; i < dk; i += 256) {
-        const float *w = P.a2 + (long long)(h * dk + i) * P.rank;
-        float z = 0.f;
-        for (int r = 0; r < P.rank; r++) z = fmaf(w[r], a1[r], z);
-        al[i] = expf(gla_log_alpha(z + P.a2b[h * dk + i], P.tau));
-    }
-    __syncthreads();
+    lds_barrier();
     f32x4 o = {};
     if (r0 < rp) {
         const f32x4 vv = *reinterpret_cast<const f32x4 *>(v + c4 * 4);
@@ -317,33 +398,36 @@ __device__ __forceinline__ void gla_decode_block(const GlaParams &P, int h, int 
         }
         *reinterpret_cast<f32x4 *>(part + r0 * P.dvp + c4 * 4) = o;
     }
-    __syncthreads();
+    lds_barrier();
     float val = 0.f;                                     // dvp <= 256: one value column per thread
-    if (tid < dv)
+    if (vc)
         for (int r = 0; r < rp; r++) val += part[r * P.dvp + tid];
     const float ss = wave_sum(val * val);
     if ((tid & 63) == 0) red[tid >> 6] = ss;
-    __syncthreads();
-    if (tid < dv) {
-        const float inv = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)dv + P.eps);
-        const float gz = pr[P.off_g + h * dv + tid];
-        put(reinterpret_cast<T *>(P.y) + op_index(n, P.y_k0 + h * dv + tid, P.y_nks), val * inv * P.norm[tid] * (gz * sigmoid_f32(gz)) * P.oscale);
+    lds_barrier();
+    if (vc) {
+        const float inv = rsqrt_f32((red[0] + red[1] + red[2] + red[3]) / (float)dv + P.eps);
+        put(reinterpret_cast<T *>(P.y) + op_index(n, P.y_k0 + h * dv + tid, P.y_nks), val * inv * nrm * (gz * sigmoid_f32(gz)));
     }
 }
 
 template <typename T, bool OUT>
 hipError_t launch_gla_seg(const GlaParams &P, int nsegs, hipStream_t st) {
-    const int nw = P.dvp / 16;
-    const size_t lds = (size_t)(3 * 16 * (P.dkp + 4) + P.dkp + 16 * 20 + nw * 256) * 4;
+    const int nw = std::max(P.dvp, P.dkp) / 16;
+    const size_t lds = (size_t)(3 * 16 * (P.dkp + 4) + P.dkp + 16 * 20 + nw * 16 + 16 + nw * 256) * 4;
     auto go = [&](auto kfn) {
         if (lds > 65536)
             if (hipError_t s = hipFuncSetAttribute(reinterpret_cast<const void *>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)) return s;
         hipLaunchKernelGGL(kfn, dim3(nsegs, P.heads), dim3(nw * 64), lds, st, P);
         return hipGetLastError();
     };
-    if (P.dkp <= 64) return go(gla_seg_kernel<T, 4, OUT>);
-    if (P.dkp <= 128) return go(gla_seg_kernel<T, 8, OUT>);
-    return go(gla_seg_kernel<T, 16, OUT>);
+    if (nw <= 8) {
+        const bool two = 16 * P.dkp <= 2 * nw * 64;
+        if (P.dkp <= 64) return two ? go(gla_seg_kernel<T, 4, 2, 8, OUT>) : go(gla_seg_kernel<T, 4, 4, 8, OUT>);
+        return go(gla_seg_kernel<T, 8, 4, 8, OUT>);        // nw <= 8: dkp <= 128
+    }
+    if (P.dkp <= 128) return go(gla_seg_kernel<T, 8, 4, 16, OUT>);
+    return go(gla_seg_kernel<T, 16, 4, 16, OUT>);
 }
 
 // the recurrence of a ragged step: runs = streams' token runs with more than one segment (their first segments in P.runs)

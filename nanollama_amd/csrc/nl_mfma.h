@@ -65,12 +65,22 @@ __device__ __forceinline__ void put4(bf16 *p, f32x4 v) {
 }
 __device__ __forceinline__ void put4(float *p, f32x4 v) { *reinterpret_cast<f32x4 *>(p) = v; }
 
+// Single-precision functions on the hardware's v_exp_f32 / v_rcp_f32 / v_rsq_f32 (1 ulp each).  exp: the rounding of x log2(e) is
+// carried as a correction, so the result stays within a few ulp for large |x| too; x finite.
+__device__ __forceinline__ float exp_f32(float x) {
+    constexpr float L = 1.44269504f, LLO = 1.92596299e-8f, LN2 = 0.693147181f;      // log2(e) = L + LLO
+    const float t = x * L, r = fmaf(x, LLO, fmaf(x, L, -t)), e = __builtin_amdgcn_exp2f(t);
+    return fmaf(e, r * LN2, e);
+}
+__device__ __forceinline__ float rcp_f32(float x) { return __builtin_amdgcn_rcpf(x); }
+__device__ __forceinline__ float rsqrt_f32(float x) { return __builtin_amdgcn_rsqf(x); }
 __device__ __forceinline__ float sigmoid_f32(float z) {
-    const float e = expf(-fabsf(z));
-    return (z >= 0.f ? 1.f : e) / (1.f + e);
+    const float e = exp_f32(-fminf(fabsf(z), 100.f)), r = rcp_f32(1.f + e);
+    return z >= 0.f ? r : e * r;
 }
 __device__ __forceinline__ float gelu_tanh_f32(float z) {
-    return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+    // 0.5 (1 + tanh u) = sigmoid(2 u)
+    return z * sigmoid_f32(1.5957691216057308f * (z + 0.044715f * z * z * z));
 }
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
@@ -84,6 +94,14 @@ __device__ __forceinline__ void lds_dma16(const void *src_lane, void *lds_base) 
                                      (__attribute__((address_space(3))) void *)lds_base, 16, 0, 0);
 }
 __device__ __forceinline__ void lds_dma_wait() { asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); }
+
+// Workgroup barrier for data that passes through LDS only.  __syncthreads() also waits for every global load and store the wavefront
+// has in flight, i.e. for exactly the prefetches that are meant to run past it.
+__device__ __forceinline__ void lds_barrier() {
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+}
 
 // ------------------------------------------------------------- upload ---
 
@@ -101,10 +119,10 @@ __global__ void pack_operand_kernel(const void *src, int src_f32, long long rows
         put(dst + op_index(((R >> 4) * tstride + toff) * 16 + (R & 15), k0 + c, nks), v);
     }
 }
-// a vector / small matrix as float, plus a constant (1 where a norm's gain is 1 + w)
-__global__ void widen_kernel(const void *src, int src_f32, long long n, float add, float *dst) {
+// a vector / small matrix as float, plus a constant (1 where a norm's gain is 1 + w); cols > 1: transposed to [cols][n / cols]
+__global__ void widen_kernel(const void *src, int src_f32, long long n, float add, float *dst, int cols) {
     for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long long)gridDim.x * blockDim.x)
-        dst[i] = (src_f32 ? reinterpret_cast<const float *>(src)[i]
+        dst[cols > 1 ? i % cols * (n / cols) + i / cols : i] = (src_f32 ? reinterpret_cast<const float *>(src)[i]
                           : __uint_as_float((unsigned)reinterpret_cast<const unsigned short *>(src)[i] << 16)) + add;
 }
 
@@ -132,33 +150,60 @@ struct NormParams {
     const float *x, *w;    // w: the factor itself
     const int *rows;       // row of x for output token n; null: n
     void *out;
-    int dim, nks;
+    int dim, nks, n_tokens;
     float eps;
 };
+// grid (tiles of 16 tokens, splits of K): every workgroup sums the squares of its 16 rows and stores its share of the k tiles, whole
+// 16-row tiles at a time (contiguous stores)
 template <typename T>
-__global__ void __launch_bounds__(256) norm_operand_kernel(NormParams P) {
-    __shared__ float red[4];
-    const int n = blockIdx.x, tid = threadIdx.x;
-    const float *x = P.x + (long long)(P.rows ? P.rows[n] : n) * P.dim;
-    float ss = 0.f;
-    for (int k = tid; k < P.dim; k += 256) ss += x[k] * x[k];
-    ss = wave_sum(ss);
-    if ((tid & 63) == 0) red[tid >> 6] = ss;
-    __syncthreads();
-    const float inv = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)P.dim + P.eps);
-    T *out = reinterpret_cast<T *>(P.out);
-    for (int k8 = tid; k8 < P.nks * 4; k8 += 256) {
-        f32x4 a, b;
+__global__ void __launch_bounds__(512) norm_operand_kernel(NormParams P) {
+    __shared__ float inv_s[16];
+    const int n0 = blockIdx.x * 16, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+    const bool vec = (P.dim & 3) == 0;
 #pragma unroll
-        for (int j = 0; j < 8; j++) {
-            const int k = k8 * 8 + j;
-            const float v = k < P.dim ? x[k] * inv * P.w[k] : 0.f;
-            if (j < 4) a[j] = v; else b[j - 4] = v;
+    for (int i = 0; i < 2; i++) {
+        const int n = min(n0 + w * 2 + i, P.n_tokens - 1);
+        const float *x = P.x + (long long)(P.rows ? P.rows[n] : n) * P.dim;
+        float ss = 0.f;
+        if (vec) {
+#pragma unroll 4
+            for (int k = lane * 4; k < P.dim; k += 256) {
+                const f32x4 v = *reinterpret_cast<const f32x4 *>(x + k);
+                ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+            }
+        } else
+            for (int k = lane; k < P.dim; k += 64) ss += x[k] * x[k];
+        ss = wave_sum(ss);
+        if (lane == 0) inv_s[w * 2 + i] = rsqrt_f32(ss / (float)P.dim + P.eps);
+    }
+    __syncthreads();
+    const int r = lane & 15, n = min(n0 + r, P.n_tokens - 1);
+    const float *x = P.x + (long long)(P.rows ? P.rows[n] : n) * P.dim;
+    const float inv = inv_s[r];
+    T *out = reinterpret_cast<T *>(P.out) + (long long)blockIdx.x * P.nks * OPT;
+    for (int ks = blockIdx.y * 8 + w; ks < P.nks; ks += gridDim.y * 8) {
+        const int k0 = ks * 32 + (lane >> 4) * 8;
+        f32x4 a, b;
+        if (vec && k0 + 8 <= P.dim) {
+            a = *reinterpret_cast<const f32x4 *>(x + k0) * inv * *reinterpret_cast<const f32x4 *>(P.w + k0);
+            b = *reinterpret_cast<const f32x4 *>(x + k0 + 4) * inv * *reinterpret_cast<const f32x4 *>(P.w + k0 + 4);
+        } else {
+#pragma unroll
+            for (int j = 0; j < 8; j++) {
+                const float v = k0 + j < P.dim ? x[k0 + j] * inv * P.w[k0 + j] : 0.f;
+                if (j < 4) a[j] = v; else b[j - 4] = v;
+            }
         }
-        T *o = out + op_index(n, k8 * 8, P.nks);
+        T *o = out + ks * OPT + lane * 8;
         put4(o, a);
         put4(o + 4, b);
     }
+}
+template <typename T>
+hipError_t launch_norm_operand(const NormParams &P, hipStream_t st) {
+    const int tt = (P.n_tokens + 15) / 16, split = std::max(1, std::min((P.nks + 7) / 8, 256 / tt));
+    hipLaunchKernelGGL(norm_operand_kernel<T>, dim3(tt, split), dim3(512), 0, st, P);
+    return hipGetLastError();
 }
 
 // ----------------------------------------------------------- products ---
@@ -176,6 +221,9 @@ struct MatParams {
     const float *nx, *nw;
     int ndim;
     float neps;
+    // one token: every row tile's largest result and its row, for the argmax that follows (or null)
+    float *amax_val;
+    int *amax_idx;
 };
 
 __device__ __forceinline__ void store_rows(float *out, int ldo, int rows, int tok, int row, f32x4 v) {
@@ -273,83 +321,138 @@ __global__ void __launch_bounds__(256) many_kernel(MatParams P) {
 }
 
 constexpr int FEW_MAX_TOKENS = 64;
-constexpr int FEW_NORM_ELEMS = 8192;      // tokens x dim up to which few_kernel computes the norm itself
-constexpr int FEW_PRE = 6;                // k tiles per wavefront and round: all their weight loads are in flight together
+constexpr int FEW_NORM_SLOTS = 16;        // (token, 512 columns) slots up to which few_kernel computes the norm itself
 
-// decode batches: one row tile (ST_GATED: a gate and an up tile) per workgroup, k tiles dealt to its wavefronts in turn
-template <typename T, int EPI, int NT, bool NORM>
-__global__ void __launch_bounds__(512) few_kernel(MatParams P) {
+// activations go round the vector L1 (sc1): they are L2-resident and every workgroup streams them once
+__device__ __forceinline__ void load_act(Frag<bf16> &f, const __amdgpu_buffer_rsrc_t rs, unsigned byte_off) {
+    f.v = __builtin_bit_cast(bf16x8, __builtin_amdgcn_raw_buffer_load_b128(rs, byte_off, 0, 16));
+}
+__device__ __forceinline__ void load_act(Frag<float> &f, const __amdgpu_buffer_rsrc_t rs, unsigned byte_off) {
+    f.a = __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(rs, byte_off, 0, 16));
+    f.b = __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(rs, byte_off + 16, 0, 16));
+}
+
+// decode batches: one row tile (ST_GATED: a gate and an up tile) x NT token tiles per workgroup, k tiles dealt to its WV wavefronts
+// in turn; a round's loads are all in flight together
+template <typename T, int EPI, int NT, int WV, bool NORM>
+__global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P) {
     constexpr int RB = EPI == ST_GATED ? 2 : 1;
+    constexpr int PRE = (NT == 1 ? 8 : NT == 2 ? 6 : WV == 16 ? 4 : 6) / (sizeof(T) == 4 ? 2 : 1);
     extern __shared__ __align__(16) char lds[];
-    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, nw = blockDim.x >> 6, g = lane >> 4, col = lane & 15;
-    const int rt = blockIdx.x * RB, nks = P.nks, n = P.n_tokens;
-    const Frag<T> *W = reinterpret_cast<const Frag<T> *>(P.W) + (long long)rt * nks * 64 + lane;
-    const Frag<T> *X = reinterpret_cast<const Frag<T> *>(P.X) + lane;
-    f32x4 acc[RB][NT] = {};
-    Frag<T> a[RB][FEW_PRE];
-    auto load_a = [&](int k0) {
+    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, col = lane & 15;
+    const int rt = blockIdx.x * RB, tt0 = blockIdx.y * NT, nks = P.nks, n = P.n_tokens;
+    // NORM: the residual rows are requested ahead of the weights (loads return in order)
+    float xv[NORM ? FEW_NORM_SLOTS : 1], wv[NORM ? FEW_NORM_SLOTS : 1];
+    const int ux = NORM ? (nks * 32 + 511) >> 9 : 1, nslots = NORM ? n * ux : 0;
+    if constexpr (NORM) {
+        int t = 0, u = 0;
 #pragma unroll
-        for (int u = 0; u < FEW_PRE; u++) {
-            const int ks = min(k0 + u * nw, nks - 1);
+        for (int s = 0; s < FEW_NORM_SLOTS; s++)
+            if (s < nslots) {
+                const int k = u * 512 + tid;
+                xv[s] = k < P.ndim ? P.nx[(long long)t * P.ndim + k] : 0.f;
+                wv[s] = k < P.ndim ? P.nw[k] : 0.f;
+                if (++u == ux) { u = 0; t++; }
+            }
+    }
+    const Frag<T> *W = reinterpret_cast<const Frag<T> *>(P.W) + (long long)rt * nks * 64 + lane;
+    const __amdgpu_buffer_rsrc_t X = __builtin_amdgcn_make_buffer_rsrc(const_cast<void *>(P.X), 0, NORM ? 0 : (int)(((n + 15) >> 4) * nks * OPT * sizeof(T)), 0x00027000);
+    f32x4 acc[RB][NT] = {};
+    Frag<T> a[RB][PRE], b[PRE][NT];
+    auto load = [&](int k0) {
+#pragma unroll
+        for (int u = 0; u < PRE; u++) {
+            const int ks = min(k0 + u * WV, nks - 1);
 #pragma unroll
             for (int r = 0; r < RB; r++) a[r][u] = W[((long long)r * nks + ks) * 64];
+            if constexpr (!NORM) {
+#pragma unroll
+                for (int t = 0; t < NT; t++) {
+                    frag_zero(b[u][t]);
+                    if ((tt0 + t) * 16 + col < n) load_act(b[u][t], X, (unsigned)((((tt0 + t) * nks + ks) * 64 + lane) * 8 * sizeof(T)));
+                }
+            }
         }
     };
-    load_a(w);
+    load(w);
     T *xs = reinterpret_cast<T *>(lds);                    // NORM: [nks][4][n][8]
     if constexpr (NORM) {
-        float *red = reinterpret_cast<float *>(lds + (size_t)nks * 32 * n * sizeof(T));
-        for (int t = 0; t < n; t++) {
-            const float *x = P.nx + (long long)t * P.ndim;
-            float ss = 0.f;
-            for (int k = tid; k < P.ndim; k += blockDim.x) ss += x[k] * x[k];
-            ss = wave_sum(ss);
-            if (lane == 0) red[t * 8 + w] = ss;
-        }
-        __syncthreads();
-        for (int t = 0; t < n; t++) {
-            const float *x = P.nx + (long long)t * P.ndim;
-            float ss = 0.f;
-            for (int q = 0; q < nw; q++) ss += red[t * 8 + q];
-            const float inv = 1.f / sqrtf(ss / (float)P.ndim + P.neps);
-            for (int k = tid; k < nks * 32; k += blockDim.x)
-                put(xs + ((k >> 3) * n + t) * 8 + (k & 7), k < P.ndim ? x[k] * inv * P.nw[k] : 0.f);
-        }
-        __syncthreads();
-    }
-    for (int k0 = w; k0 < nks; k0 += FEW_PRE * nw) {
-        if (k0 != w) load_a(k0);
+        float *red = reinterpret_cast<float *>(lds + (size_t)nks * 32 * n * sizeof(T));      // [n][WV]
+        int t = 0, u = 0;
+        float ss = 0.f;
 #pragma unroll
-        for (int u = 0; u < FEW_PRE; u++) {
-            const int ks = k0 + u * nw;
-            if (ks >= nks) break;
-#pragma unroll
-            for (int t = 0; t < NT; t++) {
-                Frag<T> b;
-                frag_zero(b);
-                if (t * 16 + col < n) {
-                    if constexpr (NORM) b = *reinterpret_cast<const Frag<T> *>(xs + ((ks * 4 + g) * n + col) * 8);
-                    else b = X[((long long)t * nks + ks) * 64];
+        for (int s = 0; s < FEW_NORM_SLOTS; s++)
+            if (s < nslots) {
+                ss += xv[s] * xv[s];
+                if (++u == ux) {
+                    ss = wave_sum(ss);
+                    if (lane == 0) red[t * WV + w] = ss;
+                    ss = 0.f; u = 0; t++;
                 }
-#pragma unroll
-                for (int r = 0; r < RB; r++) acc[r][t] = mma(a[r][u], b, acc[r][t]);
             }
+        lds_barrier();
+        float inv = 0.f;
+        t = u = 0;
+#pragma unroll
+        for (int s = 0; s < FEW_NORM_SLOTS; s++)
+            if (s < nslots) {
+                if (u == 0) {
+                    float q = 0.f;
+#pragma unroll
+                    for (int i = 0; i < WV; i++) q += red[t * WV + i];
+                    inv = rsqrt_f32(q / (float)P.ndim + P.neps);
+                }
+                const int k = u * 512 + tid;
+                if (k < nks * 32) put(xs + ((k >> 3) * n + t) * 8 + (k & 7), xv[s] * inv * wv[s]);
+                if (++u == ux) { u = 0; t++; }
+            }
+        lds_barrier();
+    }
+    for (int k0 = w; k0 < nks; k0 += PRE * WV) {
+        if (k0 != w) load(k0);
+#pragma unroll
+        for (int u = 0; u < PRE; u++) {
+            const int ks = k0 + u * WV;
+            if (ks >= nks) break;
+            if constexpr (NORM) {
+                frag_zero(b[u][0]);
+                if (col < n) b[u][0] = *reinterpret_cast<const Frag<T> *>(xs + ((ks * 4 + g) * n + col) * 8);
+            }
+#pragma unroll
+            for (int t = 0; t < NT; t++)
+#pragma unroll
+                for (int r = 0; r < RB; r++) acc[r][t] = mma(a[r][u], b[u][t], acc[r][t]);
         }
     }
     // the wavefronts' partial tiles meet in LDS
-    __syncthreads();
-    f32x4 *red = reinterpret_cast<f32x4 *>(lds);           // [nw][RB * NT][64]
+    if constexpr (NORM) lds_barrier();                   // (the area held the norm)
+    f32x4 *red = reinterpret_cast<f32x4 *>(lds);           // [WV][RB * NT][64]
 #pragma unroll
     for (int r = 0; r < RB; r++)
 #pragma unroll
         for (int t = 0; t < NT; t++) red[(w * RB * NT + r * NT + t) * 64 + lane] = acc[r][t];
-    __syncthreads();
-    for (int i = tid; i < NT * 64; i += blockDim.x) {
-        const int t = i >> 6, l = i & 63, tok = t * 16 + (l & 15), row = rt * 16 + 4 * (l >> 4);
+    lds_barrier();
+    for (int i = tid; i < NT * 64; i += WV * 64) {
+        const int t = i >> 6, l = i & 63, tok = (tt0 + t) * 16 + (l & 15), row = rt * 16 + 4 * (l >> 4);
         f32x4 v[RB] = {};
-        for (int q = 0; q < nw; q++)
+#pragma unroll
+        for (int q = 0; q < WV; q++)
 #pragma unroll
             for (int r = 0; r < RB; r++) v[r] += red[(q * RB * NT + r * NT + t) * 64 + l];
+        if (EPI == ST_F32 && NT == 1 && P.amax_val) {      // one token: rows of column 0, four lanes with four rows each
+            float best = -INFINITY;
+            int idx = 0x7fffffff;
+            if ((l & 15) == 0)
+                for (int j = 0; j < 4; j++)
+                    if (row + j < P.rows && v[0][j] > best) { best = v[0][j]; idx = row + j; }
+#pragma unroll
+            for (int o = 16; o < 64; o <<= 1) {
+                const float ov = __shfl_xor(best, o);
+                const int oi = __shfl_xor(idx, o);
+                if (ov > best || (ov == best && oi < idx)) { best = ov; idx = oi; }
+            }
+            if (l == 0) { P.amax_val[blockIdx.x] = best; P.amax_idx[blockIdx.x] = idx; }
+        }
         if (tok >= n) continue;
         if constexpr (EPI == ST_F32) store_rows(P.out, P.ldo, P.rows, tok, row, v[0]);
         else if constexpr (EPI == ST_RESID) add_rows(P.out, P.add2, P.ldo, P.rows, tok, row, v[0]);
@@ -357,30 +460,43 @@ __global__ void __launch_bounds__(512) few_kernel(MatParams P) {
     }
 }
 
-template <typename T, int EPI, int NT, bool NORM>
+template <typename T, int EPI, int NT, int WV, bool NORM>
 hipError_t launch_few_nt(const MatParams &P, hipStream_t st) {
-    const int RB = EPI == ST_GATED ? 2 : 1;
-    const int nw = NT > 2 ? 4 : 8;
-    size_t lds = (size_t)nw * RB * NT * 64 * 16;
-    if (NORM) lds = std::max(lds, (size_t)P.nks * 32 * P.n_tokens * sizeof(T) + (size_t)P.n_tokens * 8 * 4);
-    hipLaunchKernelGGL((few_kernel<T, EPI, NT, NORM>), dim3(P.nrt / RB), dim3(nw * 64), lds, st, P);
+    constexpr int RB = EPI == ST_GATED ? 2 : 1;
+    const int tt = (P.n_tokens + 15) / 16;
+    size_t lds = (size_t)WV * RB * NT * 64 * 16;           // at most 64 KB
+    if (NORM) lds = std::max(lds, (size_t)P.nks * 32 * P.n_tokens * sizeof(T) + (size_t)P.n_tokens * WV * 4);
+    hipLaunchKernelGGL((few_kernel<T, EPI, NT, WV, NORM>), dim3(P.nrt / RB, (tt + NT - 1) / NT), dim3(WV * 64), lds, st, P);
     return hipGetLastError();
 }
 // is the norm of the product's input computed inside the launch?
-inline bool few_norm_ok(int n, int dim) { return n <= 16 && (long long)n * dim <= FEW_NORM_ELEMS; }
+inline bool few_norm_ok(int n, int nks) { return n * ((nks * 32 + 511) / 512) <= FEW_NORM_SLOTS; }
+
+template <typename T, int EPI>
+hipError_t launch_few(const MatParams &P, hipStream_t st, bool norm) {
+    constexpr int RB = EPI == ST_GATED ? 2 : 1;
+    if (norm) return launch_few_nt<T, EPI, 1, 8, true>(P, st);
+    const int tt = (P.n_tokens + 15) / 16, blocks = P.nrt / RB;
+    // few row tiles: sixteen wavefronts to a workgroup, and token tiles on workgroups of their own, until the chip is covered
+    const bool deep = RB == 1 && blocks < 256 && P.nks >= 48;
+    int nt = tt >= 3 ? 4 : tt;
+    while (nt > 1 && blocks * ((tt + nt - 1) / nt) < 192) nt /= 2;
+    if constexpr (RB == 1) {
+        if (deep) {
+            if (nt == 1) return launch_few_nt<T, EPI, 1, 16, false>(P, st);
+            if (nt == 2) return launch_few_nt<T, EPI, 2, 16, false>(P, st);
+            return launch_few_nt<T, EPI, 4, 16, false>(P, st);
+        }
+    }
+    if (nt == 1) return launch_few_nt<T, EPI, 1, 8, false>(P, st);
+    if (nt == 2) return launch_few_nt<T, EPI, 2, 8, false>(P, st);
+    return launch_few_nt<T, EPI, 4, 8, false>(P, st);
+}
 
 template <typename T, int EPI>
 hipError_t launch_product(MatParams P, hipStream_t st, bool norm = false) {
     if (P.n_tokens <= 0) return hipSuccess;
-    if (P.n_tokens <= FEW_MAX_TOKENS) {
-        if (norm) return launch_few_nt<T, EPI, 1, true>(P, st);
-        switch ((P.n_tokens + 15) / 16) {
-        case 1: return launch_few_nt<T, EPI, 1, false>(P, st);
-        case 2: return launch_few_nt<T, EPI, 2, false>(P, st);
-        case 3: return launch_few_nt<T, EPI, 3, false>(P, st);
-        default: return launch_few_nt<T, EPI, 4, false>(P, st);
-        }
-    }
+    if (P.n_tokens <= FEW_MAX_TOKENS) return launch_few<T, EPI>(P, st, norm);
     const int ntb = (P.n_tokens + 127) / 128;
     auto go = [&](auto kfn, int rt) {
         const int total = (P.nrt + rt - 1) / rt * ntb;

@@ -83,6 +83,8 @@ struct nl_engine {
     void *h = nullptr, *y = nullptr, *act = nullptr, *q = nullptr;
     float *ldec = nullptr, *inc = nullptr, *totlog = nullptr, *part = nullptr;
     unsigned *arrived = nullptr;
+    float *amax_val = nullptr;   // one token's logits: the largest of every 16 rows (the argmax reads these)
+    int *amax_idx = nullptr;
     int lm_cap = 0;              // rows of `logits`
     int seg_cap = 0;
     // step metadata: pinned image and device copy of [tok | pos | stream | rows | subs | segs | tiles | runs]
@@ -142,7 +144,8 @@ struct Dest {                    // where a tensor goes
     long long rows = 0, cols = 0;
     Mat *mat = nullptr;          // operand order ...
     int row0 = 0, k0 = 0, tstride = 1, toff = 0;
-    float *vec = nullptr;        // ... or plain float, plus `add`
+    float *vec = nullptr;        // ... or plain float, plus `add`, transposed if asked for
+    bool transpose = false;
     float add = 0.f;
 };
 
@@ -174,7 +177,7 @@ bool find_dest(nl_engine *e, const char *name, Dest &d) {
         if (f == "lin.v") return in(L.lv, G.heads * G.vdim);
         if (f == "lin.g") return in(L.lg, G.heads * G.vdim);
         if (f == "lin.a1") return in(L.la1, G.rank);
-        if (f == "lin.a2") return vec(L.a2, G.heads * G.dim, G.rank, 0.f);
+        if (f == "lin.a2") { d.transpose = true; return vec(L.a2, G.heads * G.dim, G.rank, 0.f); }
         if (f == "lin.a2_bias") return vec(L.a2b, 1, G.heads * G.dim, 0.f);
         if (f == "lin.norm") return vec(L.lnorm, 1, G.vdim, 0.f);
         if (f == "lin.o") { d.mat = &L.out; d.k0 = L.y_lin; d.rows = D; d.cols = G.heads * G.vdim; return true; }
@@ -220,21 +223,23 @@ struct StepIn {                  // one launch sequence
 
 template <typename T, int EPI>
 hipError_t product(nl_engine *e, const Mat &m, const void *X, int n, float *out, int ldo, const float *add2, void *act, int act_nks,
-                   const float *nx = nullptr, const float *nw = nullptr) {
+                   const float *nx = nullptr, const float *nw = nullptr, float *amax_val = nullptr, int *amax_idx = nullptr) {
     MatParams P{};
     P.W = m.w; P.X = X; P.nks = m.nks; P.nrt = m.nrt; P.n_tokens = n; P.rows = m.rows; P.out = out; P.ldo = ldo; P.add2 = add2;
     P.act = act; P.act_nks = act_nks; P.nx = nx; P.nw = nw; P.ndim = e->c.dim; P.neps = e->c.eps;
+    P.amax_val = amax_val; P.amax_idx = amax_idx;
     return launch_product<T, EPI>(P, e->stream, nx != nullptr);
 }
 
 // B = norm(x): inside the product's launch or as an operand of its own
 template <typename T, int EPI>
-hipError_t normed_product(nl_engine *e, const Mat &m, const float *x, const int *rows, const float *nw, int n, float *out, int ldo, void *act, int act_nks) {
-    if (!rows && few_norm_ok(n, e->c.dim)) return product<T, EPI>(e, m, nullptr, n, out, ldo, nullptr, act, act_nks, x, nw);
+hipError_t normed_product(nl_engine *e, const Mat &m, const float *x, const int *rows, const float *nw, int n, float *out, int ldo, void *act, int act_nks,
+                          float *amax_val = nullptr, int *amax_idx = nullptr) {
+    if (!rows && few_norm_ok(n, m.nks)) return product<T, EPI>(e, m, nullptr, n, out, ldo, nullptr, act, act_nks, x, nw, amax_val, amax_idx);
     NormParams N{};
-    N.x = x; N.w = nw; N.rows = rows; N.out = e->h; N.dim = e->c.dim; N.nks = e->nksd; N.eps = e->c.eps;
-    hipLaunchKernelGGL(norm_operand_kernel<T>, dim3(n), dim3(256), 0, e->stream, N);
-    return product<T, EPI>(e, m, e->h, n, out, ldo, nullptr, act, act_nks);
+    N.x = x; N.w = nw; N.rows = rows; N.out = e->h; N.dim = e->c.dim; N.nks = e->nksd; N.n_tokens = n; N.eps = e->c.eps;
+    if (hipError_t s = launch_norm_operand<T>(N, e->stream)) return s;
+    return product<T, EPI>(e, m, e->h, n, out, ldo, nullptr, act, act_nks, nullptr, nullptr, amax_val, amax_idx);
 }
 
 template <typename T>
@@ -288,7 +293,8 @@ hipError_t launch_sequence(nl_engine *e, const StepIn &s) {
         }
     }
     if (s.n_out > 0)
-        return normed_product<T, ST_F32>(e, e->embed, e->x, s.rows, e->final_norm, s.n_out, s.logits, e->c.vocab, nullptr, 0);
+        return normed_product<T, ST_F32>(e, e->embed, e->x, s.rows, e->final_norm, s.n_out, s.logits, e->c.vocab, nullptr, 0,
+                                         s.n_out == 1 ? e->amax_val : nullptr, s.n_out == 1 ? e->amax_idx : nullptr);
     return hipGetLastError();
 }
 
@@ -299,13 +305,13 @@ int run_sequence(nl_engine *e, const StepIn &s) {
     return NL_OK;
 }
 
-// key-range splits of a decode step: enough workgroups for the chip, at least 128 keys each, never more keys than one split holds
+// key-range splits of a decode step: enough workgroups for the chip, at least 256 keys each, never more keys than one split holds
 int splits_for(const nl_engine *e, int n, int max_pos) {
     int out = 1;
     for (const Layer &L : e->layers) {
         if (!L.d.attn.heads) continue;
         const int seen = L.d.attn.window > 0 ? std::min(L.d.attn.window, max_pos + 1) : max_pos + 1, nb = seen / 32 + 2;
-        const int need = (nb * 32 + WA_SPLIT_KEYS - 1) / WA_SPLIT_KEYS, want = std::min(512 / std::max(1, n * L.d.attn.heads), nb / 4);
+        const int need = (nb * 32 + WA_SPLIT_KEYS - 1) / WA_SPLIT_KEYS, want = std::min(512 / std::max(1, n * L.d.attn.heads), nb / 8);
         int p = 1;
         while (p < need || (p * 2 <= want && p < 64)) p *= 2;
         out = std::max(out, p);
@@ -329,7 +335,7 @@ int queue_decode(nl_engine *e, int kind, int n, int max_pos, int steps = 1) {
             if (kind == CH_BATCH) hipLaunchKernelGGL(bargmax_kernel, dim3(n), dim3(1024), 0, e->stream, e->logits, e->c.vocab, e->ids);
             else if (kind != CH_SAMPLE) {
                 ArgmaxParams A{};
-                A.logits = e->logits; A.n = e->c.vocab; A.ctl = e->ctl; A.ids = e->ids; A.result = e->result;
+                A.logits = e->logits; A.n = e->c.vocab; A.part_val = e->amax_val; A.part_idx = e->amax_idx; A.npart = e->embed.nrt; A.ctl = e->ctl; A.ids = e->ids; A.result = e->result;
                 hipLaunchKernelGGL(argmax_kernel, dim3(1), dim3(1024), 0, e->stream, A);
             }
         }
@@ -599,7 +605,7 @@ int nl_upload_tensor(nl_handle e, const char *name, uint32_t type, const void *d
     HIPCK(e, hipMemcpy(e->stage, data, need, hipMemcpyHostToDevice));
     const long long n = d.rows * d.cols;
     const int f32 = type == NL_GGML_F32, grid = (int)std::min<long long>((n + 255) / 256, 8192);
-    if (d.vec) hipLaunchKernelGGL(widen_kernel, dim3(grid), dim3(256), 0, e->stream, e->stage, f32, n, d.add, d.vec);
+    if (d.vec) hipLaunchKernelGGL(widen_kernel, dim3(grid), dim3(256), 0, e->stream, e->stage, f32, n, d.add, d.vec, d.transpose ? (int)d.cols : 1);
     else if (e->f32()) hipLaunchKernelGGL(pack_operand_kernel<float>, dim3(grid), dim3(256), 0, e->stream, e->stage, f32, d.rows, d.cols, reinterpret_cast<float *>(d.mat->w), d.mat->nks, d.row0, d.k0, d.tstride, d.toff);
     else hipLaunchKernelGGL(pack_operand_kernel<bf16>, dim3(grid), dim3(256), 0, e->stream, e->stage, f32, d.rows, d.cols, reinterpret_cast<bf16 *>(d.mat->w), d.mat->nks, d.row0, d.k0, d.tstride, d.toff);
     HIPCK(e, hipGetLastError());
@@ -677,7 +683,8 @@ int nl_finalize(nl_handle e) {
     e->m_runs = e->m_tiles + tiles * (int)(sizeof(WinTile) / 4);
     e->m_words = e->m_runs + segs;
     if ((rc = dev_alloc(e, e->d_meta, (size_t)e->m_words * 4, bs)) || (rc = dev_alloc(e, e->ctl, CTL_WORDS * 4, bs)) ||
-        (rc = dev_alloc(e, e->ids, (size_t)std::max(e->ids_cap, e->lm_cap) * 4, bs)) || (rc = dev_alloc(e, e->result, 4, bs))) return rc;
+        (rc = dev_alloc(e, e->ids, (size_t)std::max(e->ids_cap, e->lm_cap) * 4, bs)) || (rc = dev_alloc(e, e->result, 4, bs)) ||
+        (rc = dev_alloc(e, e->amax_val, (size_t)e->embed.nrt * 4, bs)) || (rc = dev_alloc(e, e->amax_idx, (size_t)e->embed.nrt * 4, bs))) return rc;
     HIPCK(e, hipHostMalloc((void **)&e->h_meta, (size_t)e->m_words * 4, hipHostMallocDefault));
     HIPCK(e, hipHostMalloc((void **)&e->h_ctl, 64, hipHostMallocDefault));
     HIPCK(e, hipHostMalloc((void **)&e->h_ids, (size_t)std::max(e->ids_cap, e->lm_cap) * 4, hipHostMallocDefault));

@@ -80,7 +80,7 @@ __global__ void __launch_bounds__(256) win_prep_kernel(WinParams P) {
         v[i] = lane + 64 * i < P.dk ? src[lane + 64 * i] : 0.f;
         ss += v[i] * v[i];
     }
-    const float inv = nw ? 1.f / sqrtf(wave_sum(ss) / (float)P.dk + P.eps) : 1.f;
+    const float inv = nw ? rsqrt_f32(wave_sum(ss) / (float)P.dk + P.eps) : 1.f;
     T *q = reinterpret_cast<T *>(P.q) + ((long long)n * P.heads + u) * P.nks * 32;
     T *K = isq ? nullptr : ring_k<T>(P, P.stream[n], u - P.heads);
     const int slot = isq ? 0 : P.pos[n] % P.R;
@@ -94,7 +94,9 @@ __global__ void __launch_bounds__(256) win_prep_kernel(WinParams P) {
     }
 }
 
-template <typename T> __device__ __forceinline__ float soft_exp(float x) { return sizeof(T) == 2 ? __expf(x) : expf(x); }
+// scores live in units of log 2: 2^x is one instruction
+__device__ __forceinline__ float exp2_f32(float x) { return __builtin_amdgcn_exp2f(x); }
+constexpr float LOG2E = 1.4426950408889634f;
 
 // grid (tiles, heads); M bounds the key tiles (nks <= M) and value tiles (nvt <= 2 M)
 template <typename T, int M>
@@ -116,7 +118,7 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
     const int kpieces = KT / 16 * nks * (UNIT / 1024), vpieces = KT / 32 * nvt * (UNIT / 1024), stage = (kpieces + vpieces) * 1024;
     const int jhi = tl.pos0 + tl.nq - 1, jlo = max(0, tl.pos0 - win + 1), j0 = jlo / KT * KT;
     // queries of this wavefront: none of them sees keys outside [wlo, whi]
-    const int wq = min(w * 16, tl.nq - 1), whi = tl.pos0 + min(w * 16 + 15, tl.nq - 1), wlo = max(0, tl.pos0 + wq - win + 1);
+    const int wq = min(w * 16, tl.nq - 1), whi = tl.pos0 + min(w * 16 + 15, tl.nq - 1), wq0 = tl.pos0 + wq, wlo = max(0, wq0 - win + 1);
     auto issue = [&](int j, int buf) {
         const int slot = j % P.R;                        // R is a multiple of KT: a tile of keys is one contiguous run
         const char *ks = K + (long long)(slot >> 4) * nks * UNIT, *vs = V + (long long)(slot >> 5) * nvt * UNIT;
@@ -125,7 +127,12 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
     };
     f32x4 o[2 * M] = {};
     float m = -INFINITY, l = 0.f;
-    const float slope = P.slope ? P.slope[h] : 0.f;
+    const float scale = P.scale * LOG2E, slope = P.slope ? P.slope[h] * LOG2E : 0.f;
+    float off[KT / 16][4];                               // slope * (key's place in the tile)
+#pragma unroll
+    for (int a = 0; a < KT / 16; a++)
+#pragma unroll
+        for (int i = 0; i < 4; i++) off[a][i] = slope * (float)(a * 16 + 4 * g + i);
     issue(j0, 0);
     int buf = 0;
     for (int j = j0; j <= jhi; j += KT, buf ^= 1) {
@@ -134,24 +141,37 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
         if (j + KT <= jhi) issue(j + KT, buf ^ 1);
         if (j > whi || j + KT - 1 < wlo) continue;       // (every wavefront meets the barrier of every tile)
         const char *kb = lds + buf * stage, *vb = kb + kpieces * 1024;
-        f32x4 s[KT / 16];
-        float mx = m;
+        f32x4 s[KT / 16] = {};
 #pragma unroll
-        for (int a = 0; a < KT / 16; a++) {
-            s[a] = f32x4{};
+        for (int k = 0; k < M; k++)
+            if (k < nks) {
 #pragma unroll
-            for (int k = 0; k < M; k++)
-                if (k < nks) s[a] = mma(*reinterpret_cast<const Frag<T> *>(kb + (a * nks + k) * UNIT + lane * sizeof(Frag<T>)), qf[k], s[a]);
-#pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const int dist = qpos - (j + a * 16 + 4 * g + i);
-                s[a][i] = dist >= 0 && dist < win ? s[a][i] * P.scale - slope * (float)dist : -INFINITY;
-                mx = fmaxf(mx, s[a][i]);
+                for (int a = 0; a < KT / 16; a++)
+                    s[a] = mma(*reinterpret_cast<const Frag<T> *>(kb + (a * nks + k) * UNIT + lane * sizeof(Frag<T>)), qf[k], s[a]);
             }
+        const float away = slope * (float)(qpos - j);
+        float mx = m;
+        if (j + KT - 1 <= wq0 && j >= whi - win + 1) {   // every query of the wavefront sees every key of the tile
+#pragma unroll
+            for (int a = 0; a < KT / 16; a++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    s[a][i] = fmaf(s[a][i], scale, off[a][i] - away);
+                    mx = fmaxf(mx, s[a][i]);
+                }
+        } else {
+#pragma unroll
+            for (int a = 0; a < KT / 16; a++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const int dist = qpos - (j + a * 16 + 4 * g + i);
+                    s[a][i] = dist >= 0 && dist < win ? fmaf(s[a][i], scale, off[a][i] - away) : -INFINITY;
+                    mx = fmaxf(mx, s[a][i]);
+                }
         }
         mx = fmaxf(mx, __shfl_xor(mx, 16));
         mx = fmaxf(mx, __shfl_xor(mx, 32));
-        const float base = mx == -INFINITY ? 0.f : mx, corr = soft_exp<T>(m - base);
+        const float base = mx == -INFINITY ? 0.f : mx, corr = exp2_f32(m - base);
         m = mx;
         float add = 0.f;
         Frag<T> p[KT / 32];
@@ -159,7 +179,7 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
         for (int a = 0; a < KT / 16; a++)
 #pragma unroll
             for (int i = 0; i < 4; i++) {
-                const float e = soft_exp<T>(s[a][i] - base);
+                const float e = exp2_f32(s[a][i] - base);
                 add += e;
                 frag_set(p[a >> 1], (a & 1) * 4 + i, e);
             }
@@ -211,25 +231,49 @@ __device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int 
     // the split's blocks of 32 keys, at most WA_SPLIT_KEYS / 32 + 1 of them; the last block holds the new position
     const int b0 = lo >> 5, nb = (pos >> 5) - b0 + 1, per = (nb + P.nsplit - 1) / P.nsplit, bf = b0 + split * per, bl = min(bf + per, b0 + nb);
     const bool newest = bf < bl && bl == b0 + nb;
-    // wavefront 0 the query, wavefront 1 the new key, the others the new value
+    T *K = ring_k<T>(P, stream, gk), *V = ring_v<T>(P, stream, gk);
+    // wavefront 0 the query, wavefront 1 the new key, the others the new value; behind these loads the wavefront's first fragments of
+    // the ring, so that they are on their way during the norms
+    float v[WA_MAX_DIM / 64], nv[WA_MAX_DIM / 64];
+    const float *nw = w == 0 ? P.qnorm : P.knorm;
     if (w < 2) {
-        const float *src = pr + (w == 0 ? P.off_q + h * dk : P.off_k + gk * dk), *nw = w == 0 ? P.qnorm : P.knorm;
-        float v[WA_MAX_DIM / 64], ss = 0.f;
+        const float *src = pr + (w == 0 ? P.off_q + h * dk : P.off_k + gk * dk);
 #pragma unroll
         for (int i = 0; i < WA_MAX_DIM / 64; i++) {
-            v[i] = lane + 64 * i < dk ? src[lane + 64 * i] : 0.f;
-            ss += v[i] * v[i];
+            const bool in = lane + 64 * i < dk;
+            v[i] = in ? src[lane + 64 * i] : 0.f;
+            nv[i] = in && nw ? nw[lane + 64 * i] : 1.f;
         }
-        const float inv = nw ? 1.f / sqrtf(wave_sum(ss) / (float)dk + P.eps) : 1.f;
+    } else {
+#pragma unroll
+        for (int i = 0; i < WA_MAX_DIM / 128; i++) v[i] = tid - 128 + 128 * i < dv ? pr[P.off_v + gk * dv + tid - 128 + 128 * i] : 0.f;
+    }
+    constexpr int PF = 4;
+    Frag<T> kpre[PF], vpre[PF];
+    const int kt0 = 2 * bf + w;
+    {
+        const Frag<T> *kf = reinterpret_cast<const Frag<T> *>(K) + (long long)((kt0 * 16) % P.R >> 4) * nks * 64 + lane;
+#pragma unroll
+        for (int k = 0; k < PF; k++) kpre[k] = kf[min(k, nks - 1) * 64];
+#pragma unroll
+        for (int b = 0; b < PF; b++) vpre[b] = reinterpret_cast<const Frag<T> *>(V)[((long long)((min(bf + b, max(bl - 1, bf)) * 32) % P.R >> 5) * nvt + min(w, nvt - 1)) * 64 + lane];
+    }
+    if (w < 2) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < WA_MAX_DIM / 64; i++) ss += v[i] * v[i];
+        const float inv = nw ? rsqrt_f32(wave_sum(ss) / (float)dk + P.eps) : 1.f;
 #pragma unroll
         for (int i = 0; i < WA_MAX_DIM / 64; i++) {
             const int d = lane + 64 * i;
-            if (d < nks * 32) (w == 0 ? qn : kn)[d] = d < dk ? v[i] * inv * (nw ? nw[d] : 1.f) : 0.f;
+            if (d < nks * 32) (w == 0 ? qn : kn)[d] = d < dk ? v[i] * inv * nv[i] : 0.f;
         }
-    } else
-        for (int d = tid - 128; d < dv; d += 128) vn[d] = pr[P.off_v + gk * dv + d];
-    __syncthreads();
-    T *K = ring_k<T>(P, stream, gk), *V = ring_v<T>(P, stream, gk);
+    } else {
+#pragma unroll
+        for (int i = 0; i < WA_MAX_DIM / 128; i++)
+            if (tid - 128 + 128 * i < dv) vn[tid - 128 + 128 * i] = v[i];
+    }
+    lds_barrier();
     if (newest && h % gq == 0) {
         const int slot = pos % P.R;
         for (int d = tid; d < nks * 32; d += 256) put(K + ring_k_at(slot, d, nks), kn[d]);
@@ -238,13 +282,15 @@ __device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int 
     // scores: 16 keys per wavefront and round
     const float slope = P.slope ? P.slope[h] : 0.f;
     float mx = -INFINITY;
-    for (int t = 2 * bf + w; t < 2 * bl; t += 4) {
+    for (int t = kt0; t < 2 * bl; t += 4) {
         const int j = t * 16 + c;
         const Frag<T> *kf = reinterpret_cast<const Frag<T> *>(K) + (long long)((t * 16) % P.R >> 4) * nks * 64 + lane;
         float dot = 0.f;
 #pragma unroll 4
         for (int k = 0; k < nks; k++) {
-            const Frag<T> f = kf[k * 64];
+            Frag<T> f;
+            if (t == kt0 && k < PF) f = k == 0 ? kpre[0] : k == 1 ? kpre[1] : k == 2 ? kpre[2] : kpre[3];
+            else f = kf[k * 64];
             const f32x4 q0 = *reinterpret_cast<const f32x4 *>(qn + k * 32 + g * 8), q1 = *reinterpret_cast<const f32x4 *>(qn + k * 32 + g * 8 + 4);
             if (j == pos) {      // (its ring slot may not be written yet)
                 const f32x4 k0 = *reinterpret_cast<const f32x4 *>(kn + k * 32 + g * 8), k1 = *reinterpret_cast<const f32x4 *>(kn + k * 32 + g * 8 + 4);
@@ -263,18 +309,18 @@ __device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int 
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
     if (lane == 0) red[w] = mx;
-    __syncthreads();
+    lds_barrier();
     mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
     const float base = mx == -INFINITY ? 0.f : mx;
     float sum = 0.f;
     for (int i = tid; i < (bl - bf) * 32; i += 256) {
-        const float e = expf(sc[i] - base);
+        const float e = sc[i] == -INFINITY ? 0.f : exp_f32(sc[i] - base);
         sc[i] = e;
         sum += e;
     }
     sum = wave_sum(sum);
     if (lane == 0) red[4 + w] = sum;
-    __syncthreads();
+    lds_barrier();
     sum = red[4] + red[5] + red[6] + red[7];
     const float pnew = newest ? sc[pos - bf * 32] : 0.f;
     // values: a wavefront per tile of 16, lane (value c, key group g)
@@ -282,7 +328,9 @@ __device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int 
         float a = 0.f;
 #pragma unroll 4
         for (int b = bf; b < bl; b++) {
-            const Frag<T> f = reinterpret_cast<const Frag<T> *>(V)[((long long)((b * 32) % P.R >> 5) * nvt + t) * 64 + lane];
+            Frag<T> f;
+            if (t == w && b - bf < PF) f = b == bf ? vpre[0] : b == bf + 1 ? vpre[1] : b == bf + 2 ? vpre[2] : vpre[3];
+            else f = reinterpret_cast<const Frag<T> *>(V)[((long long)((b * 32) % P.R >> 5) * nvt + t) * 64 + lane];
             const float *p = sc + (b - bf) * 32 + g * 4;
             const int jb = b * 32 + g * 4;
 #pragma unroll
@@ -296,7 +344,7 @@ __device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int 
         a += __shfl_xor(a, 32);
         if (g == 0) os[t * 16 + c] = t * 16 + c < dv ? a + (newest ? pnew * vn[t * 16 + c] : 0.f) : 0.f;
     }
-    __syncthreads();
+    lds_barrier();
     T *y = reinterpret_cast<T *>(P.y);
     auto finish = [&](int d, float val) {
         const float gate = P.off_g < 0 ? 1.f : sigmoid_f32(pr[P.off_g + h * dv + d]);
