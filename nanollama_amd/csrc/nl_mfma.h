@@ -11,7 +11,7 @@
 // [token][in] the B operand (rows = tokens); the accumulator of a 16 x 16 tile has D[row = 4 (lane / 16) + i][token = lane % 16],
 // so a lane ends up with four consecutive outputs of one token.
 //
-// Two kernels: many_kernel for prompts (a 128 x 128 tile per workgroup, LDS double buffer filled by LDS-DMA) and few_kernel for
+// Two kernels: many_kernel for prompts (a 128 x 128 tile per workgroup, an LDS ring filled by LDS-DMA) and few_kernel for
 // decode batches of up to 64 tokens (one row tile per workgroup, K split over its wavefronts, the weights read once straight into
 // registers; for a handful of tokens the RMS norm of the layer's input runs in its prologue).  Epilogues: plain 32-bit store,
 // residual add (+ an optional second addend), gelu_tanh(gate) * up stored as the next product's operand.
@@ -93,7 +93,8 @@ __device__ __forceinline__ void lds_dma16(const void *src_lane, void *lds_base) 
     __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void *)src_lane,
                                      (__attribute__((address_space(3))) void *)lds_base, 16, 0, 0);
 }
-__device__ __forceinline__ void lds_dma_wait() { asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); }
+// until at most N of this wavefront's vector memory operations are in flight (they complete in order)
+template <int N> __device__ __forceinline__ void vm_wait() { asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory"); }
 
 // Workgroup barrier for data that passes through LDS only.  __syncthreads() also waits for every global load and store the wavefront
 // has in flight, i.e. for exactly the prefetches that are meant to run past it.
@@ -252,12 +253,15 @@ __device__ __forceinline__ void store_gated(const MatParams &P, int tok, int f16
     put4(reinterpret_cast<T *>(P.act) + op_index(tok, f16 * 16 + 4 * g, P.act_nks), v);
 }
 
-// prompts: RTW row tiles x 4 token tiles per wavefront, 2 x 2 wavefronts
+// prompts: RTW row tiles x 4 token tiles per wavefront, 2 x 2 wavefronts; the k tiles travel through a ring of LDS stages
+template <typename T, int RTW> struct ManyGeom {
+    static constexpr int RT = 2 * RTW, NT = 8, UNIT = OPT * sizeof(T), NST = sizeof(T) == 2 ? 4 : 2, STAGE = (RT + NT) * UNIT, LDS = NST * STAGE;   // 48 or 64 KB
+};
 template <typename T, int EPI, int RTW>
 __global__ void __launch_bounds__(256) many_kernel(MatParams P) {
-    constexpr int KS = sizeof(T) == 2 ? 2 : 1;             // k tiles per stage
-    constexpr int RT = 2 * RTW, NT = 8, UNIT = OPT * sizeof(T);
-    constexpr int STAGE = (RT + NT) * KS * UNIT;
+    using G = ManyGeom<T, RTW>;
+    constexpr int RT = G::RT, NT = G::NT, UNIT = G::UNIT, NST = G::NST, STAGE = G::STAGE;
+    constexpr int PW = STAGE / 4096;                       // 1 KiB pieces per stage and wavefront
     extern __shared__ __align__(16) char lds[];
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, g = lane >> 4;
     const int nrb = (P.nrt + RT - 1) / RT, ntt = (P.n_tokens + 15) >> 4, ntb = (ntt + NT - 1) / NT, total = nrb * ntb;
@@ -266,40 +270,38 @@ __global__ void __launch_bounds__(256) many_kernel(MatParams P) {
     const int per = (total + 7) / 8, id = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
     if ((int)(blockIdx.x >> 3) >= per || id >= total) return;
     const int rb = id / ntb, tb = id - rb * ntb;
-    const char *W = reinterpret_cast<const char *>(P.W), *X = reinterpret_cast<const char *>(P.X);
-    const int wr = w & 1, wt = w >> 1;
+    const int wr = w & 1, wt = w >> 1, nks = P.nks;
     f32x4 acc[RTW][4] = {};
-    constexpr int NU = (RT + NT) * KS * (UNIT / 1024);     // 1 KiB pieces per stage
-    auto issue = [&](int ks0, int buf) {
+    const char *src[PW];                                   // this wavefront's pieces of k tile 0
 #pragma unroll
-        for (int u0 = 0; u0 < NU; u0 += 4) {
-            const int u = u0 + w, piece = u % (UNIT / 1024), tile = u / (UNIT / 1024), kk = tile % KS, t = tile / KS;
-            const int ks = min(ks0 + kk, P.nks - 1);
-            const char *src = t < RT ? W + ((long long)min(rb * RT + t, P.nrt - 1) * P.nks + ks) * UNIT
-                                     : X + ((long long)min(tb * NT + t - RT, ntt - 1) * P.nks + ks) * UNIT;
-            lds_dma16(src + piece * 1024 + lane * 16, lds + buf * STAGE + u * 1024);
-        }
+    for (int i = 0; i < PW; i++) {
+        const int u = i * 4 + w, t = u / (UNIT / 1024), piece = u % (UNIT / 1024);
+        src[i] = (t < RT ? reinterpret_cast<const char *>(P.W) + (long long)min(rb * RT + t, P.nrt - 1) * nks * UNIT
+                         : reinterpret_cast<const char *>(P.X) + (long long)min(tb * NT + t - RT, ntt - 1) * nks * UNIT) + piece * 1024 + lane * 16;
+    }
+    auto issue = [&](int ks, int st) {
+#pragma unroll
+        for (int i = 0; i < PW; i++) lds_dma16(src[i] + (long long)ks * UNIT, lds + st * STAGE + (i * 4 + w) * 1024);
     };
-    issue(0, 0);
-    int buf = 0;
-    for (int ks0 = 0; ks0 < P.nks; ks0 += KS, buf ^= 1) {
-        lds_dma_wait();
-        __syncthreads();
-        if (ks0 + KS < P.nks) issue(ks0 + KS, buf ^ 1);
-        const char *base = lds + buf * STAGE;
 #pragma unroll
-        for (int kk = 0; kk < KS; kk++) {
-            if (KS > 1 && ks0 + kk >= P.nks) break;
-            Frag<T> b[4];
+    for (int s = 0; s < NST - 1; s++)
+        if (s < nks) issue(s, s);
+    int st = 0;
+    for (int ks = 0; ks < nks; ks++) {
+        if (nks - 1 - ks >= NST - 2) vm_wait<PW *(NST - 2)>();
+        else vm_wait<0>();
+        lds_barrier();
+        if (ks + NST - 1 < nks) issue(ks + NST - 1, st == 0 ? NST - 1 : st - 1);
+        const char *base = lds + st * STAGE + lane * sizeof(Frag<T>);
+        st = st + 1 == NST ? 0 : st + 1;
+        Frag<T> b[4];
 #pragma unroll
-            for (int t = 0; t < 4; t++)
-                b[t] = *reinterpret_cast<const Frag<T> *>(base + ((RT + wt * 4 + t) * KS + kk) * UNIT + lane * sizeof(Frag<T>));
+        for (int t = 0; t < 4; t++) b[t] = *reinterpret_cast<const Frag<T> *>(base + (RT + wt * 4 + t) * UNIT);
 #pragma unroll
-            for (int r = 0; r < RTW; r++) {
-                const Frag<T> a = *reinterpret_cast<const Frag<T> *>(base + ((wr * RTW + r) * KS + kk) * UNIT + lane * sizeof(Frag<T>));
+        for (int r = 0; r < RTW; r++) {
+            const Frag<T> a = *reinterpret_cast<const Frag<T> *>(base + (wr * RTW + r) * UNIT);
 #pragma unroll
-                for (int t = 0; t < 4; t++) acc[r][t] = mma(a, b[t], acc[r][t]);
-            }
+            for (int t = 0; t < 4; t++) acc[r][t] = mma(a, b[t], acc[r][t]);
         }
     }
 #pragma unroll
@@ -498,14 +500,13 @@ hipError_t launch_product(MatParams P, hipStream_t st, bool norm = false) {
     if (P.n_tokens <= 0) return hipSuccess;
     if (P.n_tokens <= FEW_MAX_TOKENS) return launch_few<T, EPI>(P, st, norm);
     const int ntb = (P.n_tokens + 127) / 128;
-    auto go = [&](auto kfn, int rt) {
+    auto go = [&](auto kfn, int rt, int lds) {
         const int total = (P.nrt + rt - 1) / rt * ntb;
-        const size_t lds = 2 * (size_t)(rt + 8) * (sizeof(T) == 2 ? 2 : 1) * OPT * sizeof(T);     // 48 or 64 KB
         hipLaunchKernelGGL(kfn, dim3((total + 7) / 8 * 8), dim3(256), lds, st, P);
         return hipGetLastError();
     };
-    if ((P.nrt + 7) / 8 * ntb >= 512) return go(many_kernel<T, EPI, 4>, 8);
-    return go(many_kernel<T, EPI, 2>, 4);
+    if ((P.nrt + 7) / 8 * ntb >= 512) return go(many_kernel<T, EPI, 4>, 8, ManyGeom<T, 4>::LDS);
+    return go(many_kernel<T, EPI, 2>, 4, ManyGeom<T, 2>::LDS);
 }
 
 }  // namespace nl

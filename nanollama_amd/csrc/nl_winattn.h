@@ -13,7 +13,7 @@
 // without leaving their lanes.  Reset is O(1): slots of another request are never visible (the mask is by position).
 //
 // PROMPTS: win_prep_kernel (norms, ring store, queries), win_attn_kernel (64 queries x one head per workgroup, keys and values
-// through LDS by LDS-DMA, double buffered).  DECODE: mix_decode_kernel -- attention heads (optionally split over key ranges, the
+// through LDS by LDS-DMA, a ring of stages).  DECODE: mix_decode_kernel -- attention heads (optionally split over key ranges, the
 // last split to arrive merges) and the linear-attention heads of a parallel layer in one launch.
 #pragma once
 #include "nl_linattn.h"
@@ -98,32 +98,40 @@ __global__ void __launch_bounds__(256) win_prep_kernel(WinParams P) {
 __device__ __forceinline__ float exp2_f32(float x) { return __builtin_amdgcn_exp2f(x); }
 constexpr float LOG2E = 1.4426950408889634f;
 
-// grid (tiles, heads); M bounds the key tiles (nks <= M) and value tiles (nvt <= 2 M)
-template <typename T, int M>
+// keys per stage, stages in the LDS ring, 1 KiB pieces a wavefront fetches per stage (a stage holds at most 8 M of them)
+template <typename T, int M> struct WinGeom {
+    static constexpr int KT = sizeof(T) == 2 ? 64 : 32, NST = M <= 2 ? 4 : M <= 4 ? 3 : 2, PW = 2 * M;
+};
+
+// grid (tiles, heads); M bounds the key tiles (nks <= M) and value tiles (nvt <= 2 M), FULL: both are equal to their bound
+template <typename T, int M, bool FULL>
 __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
-    constexpr int KT = sizeof(T) == 2 ? 64 : 32, UNIT = OPT * sizeof(T);
+    constexpr int KT = WinGeom<T, M>::KT, UNIT = OPT * sizeof(T), NST = WinGeom<T, M>::NST, PW = WinGeom<T, M>::PW;
     extern __shared__ __align__(16) char lds[];
     const WinTile tl = P.tiles[blockIdx.x];
     const int h = blockIdx.y, gk = h / (P.heads / P.kv_heads), tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, c = lane & 15;
-    const int nks = P.nks, nvt = P.nvt, qi = w * 16 + c, tok = tl.tok0 + min(qi, tl.nq - 1), qpos = tl.pos0 + min(qi, tl.nq - 1);
+    const int nks = FULL ? M : P.nks, nvt = FULL ? 2 * M : P.nvt, qi = w * 16 + c, tok = tl.tok0 + min(qi, tl.nq - 1), qpos = tl.pos0 + min(qi, tl.nq - 1);
     const int win = P.window > 0 ? P.window : 0x7fffffff;
     Frag<T> qf[M];
     {
         const T *q = reinterpret_cast<const T *>(P.q) + ((long long)tok * P.heads + h) * nks * 32 + g * 8;
 #pragma unroll
         for (int k = 0; k < M; k++)
-            if (k < nks) qf[k] = *reinterpret_cast<const Frag<T> *>(q + k * 32);
+            if (FULL || k < nks) qf[k] = *reinterpret_cast<const Frag<T> *>(q + k * 32);
     }
     const char *K = reinterpret_cast<const char *>(ring_k<T>(P, tl.stream, gk)), *V = reinterpret_cast<const char *>(ring_v<T>(P, tl.stream, gk));
     const int kpieces = KT / 16 * nks * (UNIT / 1024), vpieces = KT / 32 * nvt * (UNIT / 1024), stage = (kpieces + vpieces) * 1024;
     const int jhi = tl.pos0 + tl.nq - 1, jlo = max(0, tl.pos0 - win + 1), j0 = jlo / KT * KT;
     // queries of this wavefront: none of them sees keys outside [wlo, whi]
     const int wq = min(w * 16, tl.nq - 1), whi = tl.pos0 + min(w * 16 + 15, tl.nq - 1), wq0 = tl.pos0 + wq, wlo = max(0, wq0 - win + 1);
-    auto issue = [&](int j, int buf) {
+    auto issue = [&](int j, int st) {
         const int slot = j % P.R;                        // R is a multiple of KT: a tile of keys is one contiguous run
-        const char *ks = K + (long long)(slot >> 4) * nks * UNIT, *vs = V + (long long)(slot >> 5) * nvt * UNIT;
-        for (int u = w; u < kpieces + vpieces; u += 4)
-            lds_dma16((u < kpieces ? ks + u * 1024 : vs + (u - kpieces) * 1024) + lane * 16, lds + buf * stage + u * 1024);
+        const char *ks = K + (long long)(slot >> 4) * nks * UNIT + lane * 16, *vs = V + (long long)(slot >> 5) * nvt * UNIT + lane * 16;
+#pragma unroll
+        for (int i = 0; i < PW; i++) {                   // (the same number for every wavefront: pieces past the end repeat the last one)
+            const int u = FULL ? i * 4 + w : min(i * 4 + w, kpieces + vpieces - 1);
+            lds_dma16(u < kpieces ? ks + u * 1024 : vs + (u - kpieces) * 1024, lds + st * stage + u * 1024);
+        }
     };
     f32x4 o[2 * M] = {};
     float m = -INFINITY, l = 0.f;
@@ -133,18 +141,22 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
     for (int a = 0; a < KT / 16; a++)
 #pragma unroll
         for (int i = 0; i < 4; i++) off[a][i] = slope * (float)(a * 16 + 4 * g + i);
-    issue(j0, 0);
-    int buf = 0;
-    for (int j = j0; j <= jhi; j += KT, buf ^= 1) {
-        lds_dma_wait();
-        __syncthreads();
-        if (j + KT <= jhi) issue(j + KT, buf ^ 1);
+#pragma unroll
+    for (int i = 0; i < NST - 1; i++)
+        if (j0 + i * KT <= jhi) issue(j0 + i * KT, i);
+    int st = NST - 1;
+    for (int j = j0; j <= jhi; j += KT) {
+        if (jhi - j >= (NST - 2) * KT) vm_wait<PW *(NST - 2)>();
+        else vm_wait<0>();
+        lds_barrier();
+        if (j + (NST - 1) * KT <= jhi) issue(j + (NST - 1) * KT, st);
+        st = st + 1 == NST ? 0 : st + 1;                 // (now the current tile's stage)
         if (j > whi || j + KT - 1 < wlo) continue;       // (every wavefront meets the barrier of every tile)
-        const char *kb = lds + buf * stage, *vb = kb + kpieces * 1024;
+        const char *kb = lds + st * stage, *vb = kb + kpieces * 1024;
         f32x4 s[KT / 16] = {};
 #pragma unroll
         for (int k = 0; k < M; k++)
-            if (k < nks) {
+            if (FULL || k < nks) {
 #pragma unroll
                 for (int a = 0; a < KT / 16; a++)
                     s[a] = mma(*reinterpret_cast<const Frag<T> *>(kb + (a * nks + k) * UNIT + lane * sizeof(Frag<T>)), qf[k], s[a]);
@@ -186,7 +198,7 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
         l = l * corr + add;
 #pragma unroll
         for (int t = 0; t < 2 * M; t++)
-            if (t < nvt) {
+            if (FULL || t < nvt) {
                 o[t] *= corr;
 #pragma unroll
                 for (int b = 0; b < KT / 32; b++)
@@ -201,7 +213,7 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
     const float *gz = P.proj + (long long)tok * P.ldp + P.off_g + h * P.dv;
 #pragma unroll
     for (int t = 0; t < 2 * M; t++)
-        if (t < nvt) {
+        if (FULL || t < nvt) {
             const int d = t * 16 + 4 * g, k = P.y_k0 + h * P.dv + d;
             if (d + 3 < P.dv && (k & 3) == 0) {
                 f32x4 r;
@@ -406,8 +418,9 @@ hipError_t launch_mix_decode(const WinParams &A, const GlaParams &L, int n, hipS
 template <typename T>
 hipError_t launch_win_attn(const WinParams &P, int n_tokens, int ntiles, hipStream_t st) {
     hipLaunchKernelGGL(win_prep_kernel<T>, dim3(n_tokens, (P.heads + 2 * P.kv_heads + 3) / 4), dim3(256), 0, st, P);
-    const size_t lds = 2 * (size_t)((sizeof(T) == 2 ? 4 : 2) * P.nks + (sizeof(T) == 2 ? 2 : 1) * P.nvt) * OPT * sizeof(T);
-    auto go = [&](auto kfn) {
+    const size_t stage = (size_t)((sizeof(T) == 2 ? 4 : 2) * P.nks + (sizeof(T) == 2 ? 2 : 1) * P.nvt) * OPT * sizeof(T);
+    auto go = [&](auto kfn, int stages) {
+        const size_t lds = stages * stage;
         // (more than 64 KB of LDS needs the attribute; cheap enough to set at every such launch)
         if (lds > 65536)
             if (hipError_t s = hipFuncSetAttribute(reinterpret_cast<const void *>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)) return s;
@@ -415,11 +428,12 @@ hipError_t launch_win_attn(const WinParams &P, int n_tokens, int ntiles, hipStre
         return hipGetLastError();
     };
     const int m = std::max(P.nks, (P.nvt + 1) / 2);
-    if (m <= 1) return go(win_attn_kernel<T, 1>);
-    if (m <= 2) return go(win_attn_kernel<T, 2>);
-    if (m <= 3) return go(win_attn_kernel<T, 3>);
-    if (m <= 4) return go(win_attn_kernel<T, 4>);
-    return go(win_attn_kernel<T, 8>);
+    const bool full = P.nvt == 2 * P.nks;
+    if (m <= 1) return go(win_attn_kernel<T, 1, false>, WinGeom<T, 1>::NST);
+    if (m <= 2) return full && m == 2 ? go(win_attn_kernel<T, 2, true>, WinGeom<T, 2>::NST) : go(win_attn_kernel<T, 2, false>, WinGeom<T, 2>::NST);
+    if (m <= 3) return go(win_attn_kernel<T, 3, false>, WinGeom<T, 3>::NST);
+    if (m <= 4) return full && m == 4 ? go(win_attn_kernel<T, 4, true>, WinGeom<T, 4>::NST) : go(win_attn_kernel<T, 4, false>, WinGeom<T, 4>::NST);
+    return go(win_attn_kernel<T, 8, false>, WinGeom<T, 8>::NST);
 }
 
 }  // namespace nl
