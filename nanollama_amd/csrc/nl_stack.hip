@@ -305,13 +305,13 @@ int run_sequence(nl_engine *e, const StepIn &s) {
     return NL_OK;
 }
 
-// key-range splits of a decode step: enough workgroups for the chip, at least 256 keys each, never more keys than one split holds
+// key-range splits of a decode step: enough workgroups for the chip, at least 128 keys each, never more keys than one split holds
 int splits_for(const nl_engine *e, int n, int max_pos) {
     int out = 1;
     for (const Layer &L : e->layers) {
         if (!L.d.attn.heads) continue;
         const int seen = L.d.attn.window > 0 ? std::min(L.d.attn.window, max_pos + 1) : max_pos + 1, nb = seen / 32 + 2;
-        const int need = (nb * 32 + WA_SPLIT_KEYS - 1) / WA_SPLIT_KEYS, want = std::min(512 / std::max(1, n * L.d.attn.heads), nb / 8);
+        const int need = (nb * 32 + WA_SPLIT_KEYS - 1) / WA_SPLIT_KEYS, want = std::min(512 / std::max(1, n * L.d.attn.heads), nb / 4);
         int p = 1;
         while (p < need || (p * 2 <= want && p < 64)) p *= 2;
         out = std::max(out, p);

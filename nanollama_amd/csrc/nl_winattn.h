@@ -232,20 +232,22 @@ __host__ __device__ inline size_t win_decode_lds(int nks, int nvt) {
     return (size_t)(2 * nks * 32 + 2 * nvt * 16 + WA_SPLIT_KEYS + 64 + 16) * 4;
 }
 
-// one (head, key split, token of the batch) by a workgroup of 256
-template <typename T>
+// one (head, key split, token of the batch) by a workgroup of 256; nks <= M.  The ring's first round of keys (TB tiles of 16 per
+// wavefront) and values (VB blocks of 32) is requested before the norms: a split of 16 TB * 4 keys is one memory round trip.
+template <typename T, int M>
 __device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int split, int n, int stream, int pos, char *lds) {
+    constexpr int W = sizeof(T) == 2 ? 8 : 4, TB = W / M > 0 ? W / M : 1, VB = W;
     const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, c = lane & 15, dk = P.dk, dv = P.dv, nks = P.nks, nvt = P.nvt;
     const int gq = P.heads / P.kv_heads, gk = h / gq;
     float *qn = reinterpret_cast<float *>(lds), *kn = qn + nks * 32, *vn = kn + nks * 32, *os = vn + nvt * 16, *sc = os + nvt * 16, *red = sc + WA_SPLIT_KEYS + 64;
     const float *pr = P.proj + (long long)n * P.ldp;
     const int win = P.window > 0 ? P.window : 0x7fffffff, lo = max(0, pos - win + 1);
-    // the split's blocks of 32 keys, at most WA_SPLIT_KEYS / 32 + 1 of them; the last block holds the new position
+    // the split's blocks of 32 keys, at most WA_SPLIT_KEYS / 32 + 2 of them; the last block holds the new position
     const int b0 = lo >> 5, nb = (pos >> 5) - b0 + 1, per = (nb + P.nsplit - 1) / P.nsplit, bf = b0 + split * per, bl = min(bf + per, b0 + nb);
     const bool newest = bf < bl && bl == b0 + nb;
     T *K = ring_k<T>(P, stream, gk), *V = ring_v<T>(P, stream, gk);
-    // wavefront 0 the query, wavefront 1 the new key, the others the new value; behind these loads the wavefront's first fragments of
-    // the ring, so that they are on their way during the norms
+    const Frag<T> *Kf = reinterpret_cast<const Frag<T> *>(K) + lane, *Vf = reinterpret_cast<const Frag<T> *>(V) + lane;
+    // wavefront 0 the query, wavefront 1 the new key, the others the new value
     float v[WA_MAX_DIM / 64], nv[WA_MAX_DIM / 64];
     const float *nw = w == 0 ? P.qnorm : P.knorm;
     if (w < 2) {
@@ -260,16 +262,23 @@ __device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int 
 #pragma unroll
         for (int i = 0; i < WA_MAX_DIM / 128; i++) v[i] = tid - 128 + 128 * i < dv ? pr[P.off_v + gk * dv + tid - 128 + 128 * i] : 0.f;
     }
-    constexpr int PF = 4;
-    Frag<T> kpre[PF], vpre[PF];
+    const float gate = P.off_g >= 0 && tid < dv ? pr[P.off_g + h * dv + tid] : 0.f;      // (dv <= 256)
+    Frag<T> kf[TB][M], vf[VB];
+    auto load_keys = [&](int t0) {                       // tiles t0, t0 + 4, ...
+#pragma unroll
+        for (int i = 0; i < TB; i++)
+#pragma unroll
+            for (int k = 0; k < M; k++)
+                if (t0 + 4 * i < 2 * bl && k < nks) kf[i][k] = Kf[(long long)(((t0 + 4 * i) * 16 % P.R >> 4) * nks + k) * 64];
+    };
+    auto load_values = [&](int t, int bb) {
+#pragma unroll
+        for (int i = 0; i < VB; i++)
+            if (bb + i < bl) vf[i] = Vf[(long long)(((bb + i) * 32 % P.R >> 5) * nvt + t) * 64];
+    };
     const int kt0 = 2 * bf + w;
-    {
-        const Frag<T> *kf = reinterpret_cast<const Frag<T> *>(K) + (long long)((kt0 * 16) % P.R >> 4) * nks * 64 + lane;
-#pragma unroll
-        for (int k = 0; k < PF; k++) kpre[k] = kf[min(k, nks - 1) * 64];
-#pragma unroll
-        for (int b = 0; b < PF; b++) vpre[b] = reinterpret_cast<const Frag<T> *>(V)[((long long)((min(bf + b, max(bl - 1, bf)) * 32) % P.R >> 5) * nvt + min(w, nvt - 1)) * 64 + lane];
-    }
+    load_keys(kt0);
+    if (w < nvt) load_values(w, bf);
     if (w < 2) {
         float ss = 0.f;
 #pragma unroll
@@ -291,32 +300,36 @@ __device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int 
         for (int d = tid; d < nks * 32; d += 256) put(K + ring_k_at(slot, d, nks), kn[d]);
         for (int d = tid; d < dv; d += 256) put(V + ring_v_at(slot, d, nvt), vn[d]);
     }
-    // scores: 16 keys per wavefront and round
     const float slope = P.slope ? P.slope[h] : 0.f;
     float mx = -INFINITY;
-    for (int t = kt0; t < 2 * bl; t += 4) {
-        const int j = t * 16 + c;
-        const Frag<T> *kf = reinterpret_cast<const Frag<T> *>(K) + (long long)((t * 16) % P.R >> 4) * nks * 64 + lane;
-        float dot = 0.f;
-#pragma unroll 4
-        for (int k = 0; k < nks; k++) {
-            Frag<T> f;
-            if (t == kt0 && k < PF) f = k == 0 ? kpre[0] : k == 1 ? kpre[1] : k == 2 ? kpre[2] : kpre[3];
-            else f = kf[k * 64];
-            const f32x4 q0 = *reinterpret_cast<const f32x4 *>(qn + k * 32 + g * 8), q1 = *reinterpret_cast<const f32x4 *>(qn + k * 32 + g * 8 + 4);
-            if (j == pos) {      // (its ring slot may not be written yet)
-                const f32x4 k0 = *reinterpret_cast<const f32x4 *>(kn + k * 32 + g * 8), k1 = *reinterpret_cast<const f32x4 *>(kn + k * 32 + g * 8 + 4);
+    for (int t0 = kt0; t0 < 2 * bl; t0 += 4 * TB) {
+        if (t0 != kt0) load_keys(t0);
+        float dot[TB] = {};
 #pragma unroll
-                for (int i = 0; i < 4; i++) dot = fmaf(k1[i], q1[i], fmaf(k0[i], q0[i], dot));
-            } else
+        for (int k = 0; k < M; k++)
+            if (k < nks) {
+                const f32x4 q0 = *reinterpret_cast<const f32x4 *>(qn + k * 32 + g * 8), q1 = *reinterpret_cast<const f32x4 *>(qn + k * 32 + g * 8 + 4);
 #pragma unroll
-                for (int i = 0; i < 4; i++) dot = fmaf(frag_get(f, 4 + i), q1[i], fmaf(frag_get(f, i), q0[i], dot));
+                for (int i = 0; i < TB; i++)
+#pragma unroll
+                    for (int x = 0; x < 4; x++) dot[i] = fmaf(frag_get(kf[i][k], 4 + x), q1[x], fmaf(frag_get(kf[i][k], x), q0[x], dot[i]));
+            }
+#pragma unroll
+        for (int i = 0; i < TB; i++) {
+            const int t = t0 + 4 * i, j = t * 16 + c;
+            if (t >= 2 * bl) break;
+            if (j == pos) {                              // the new key: from this step's projection, not from the ring
+                dot[i] = 0.f;
+                for (int x = g * 8; x < nks * 32; x += 32)
+#pragma unroll
+                    for (int y = 0; y < 8; y++) dot[i] = fmaf(kn[x + y], qn[x + y], dot[i]);
+            }
+            dot[i] += __shfl_xor(dot[i], 16);
+            dot[i] += __shfl_xor(dot[i], 32);
+            const float s = j >= lo && j <= pos ? dot[i] * P.scale - slope * (float)(pos - j) : -INFINITY;
+            if (g == 0) sc[j - bf * 32] = s;
+            mx = fmaxf(mx, s);
         }
-        dot += __shfl_xor(dot, 16);
-        dot += __shfl_xor(dot, 32);
-        const float s = j >= lo && j <= pos ? dot * P.scale - slope * (float)(pos - j) : -INFINITY;
-        if (g == 0) sc[j - bf * 32] = s;
-        mx = fmaxf(mx, s);
     }
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
@@ -338,18 +351,19 @@ __device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int 
     // values: a wavefront per tile of 16, lane (value c, key group g)
     for (int t = w; t < nvt; t += 4) {
         float a = 0.f;
-#pragma unroll 4
-        for (int b = bf; b < bl; b++) {
-            Frag<T> f;
-            if (t == w && b - bf < PF) f = b == bf ? vpre[0] : b == bf + 1 ? vpre[1] : b == bf + 2 ? vpre[2] : vpre[3];
-            else f = reinterpret_cast<const Frag<T> *>(V)[((long long)((b * 32) % P.R >> 5) * nvt + t) * 64 + lane];
-            const float *p = sc + (b - bf) * 32 + g * 4;
-            const int jb = b * 32 + g * 4;
+        for (int bb = bf; bb < bl; bb += VB) {
+            if (t != w || bb != bf) load_values(t, bb);
 #pragma unroll
-            for (int i = 0; i < 4; i++) {
-                // keys outside the window weigh 0; the new key's value comes from this step's projection, not from the ring
-                const float v0 = jb + i == pos ? 0.f : frag_get(f, i), v1 = jb + 16 + i == pos ? 0.f : frag_get(f, 4 + i);
-                a = fmaf(p[16 + i], v1, fmaf(p[i], v0, a));
+            for (int i = 0; i < VB; i++) {
+                if (bb + i >= bl) break;
+                const f32x4 p0 = *reinterpret_cast<const f32x4 *>(sc + (bb + i - bf) * 32 + g * 4), p1 = *reinterpret_cast<const f32x4 *>(sc + (bb + i - bf) * 32 + g * 4 + 16);
+                const int jb = (bb + i) * 32 + g * 4;
+#pragma unroll
+                for (int x = 0; x < 4; x++) {
+                    // keys outside the window weigh 0; the new key's value comes from this step's projection, not from the ring
+                    const float v0 = jb + x == pos ? 0.f : frag_get(vf[i], x), v1 = jb + 16 + x == pos ? 0.f : frag_get(vf[i], 4 + x);
+                    a = fmaf(p1[x], v1, fmaf(p0[x], v0, a));
+                }
             }
         }
         a += __shfl_xor(a, 16);
@@ -358,52 +372,71 @@ __device__ __forceinline__ void win_decode_block(const WinParams &P, int h, int 
     }
     lds_barrier();
     T *y = reinterpret_cast<T *>(P.y);
-    auto finish = [&](int d, float val) {
-        const float gate = P.off_g < 0 ? 1.f : sigmoid_f32(pr[P.off_g + h * dv + d]);
-        put(y + op_index(n, P.y_k0 + h * dv + d, P.y_nks), val * gate * P.oscale);
+    auto finish = [&](float val) {                       // value column tid
+        put(y + op_index(n, P.y_k0 + h * dv + tid, P.y_nks), val * (P.off_g < 0 ? 1.f : sigmoid_f32(gate)) * P.oscale);
     };
     if (P.nsplit == 1) {
-        for (int d = tid; d < dv; d += 256) finish(d, os[d] / sum);
+        if (tid < dv) finish(os[tid] / sum);
         return;
     }
-    // several splits: every one leaves (max, sum, unnormalised values); the last to arrive merges, nobody waits
+    // Several splits: every one leaves (max, sum, unnormalised values); the last to arrive merges, nobody waits.  Everything that
+    // crosses workgroups goes by agent-scope accesses (past the XCD's own L2), so "stored" is the wavefront's own counter at zero:
+    // no cache is written back.
     float *mine = P.part + (((long long)n * P.heads + h) * P.nsplit + split) * (dv + 2);
-    for (int d = tid; d < dv; d += 256) __hip_atomic_store(mine + 2 + d, os[d], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    if (tid < dv) __hip_atomic_store(mine + 2 + tid, os[tid], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     if (tid == 0) {
         __hip_atomic_store(mine, mx, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
         __hip_atomic_store(mine + 1, sum, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     }
-    __threadfence();
-    __syncthreads();
+    vm_wait<0>();
+    lds_barrier();
     unsigned *arr = P.arrived + n * P.heads + h;
     unsigned *last = reinterpret_cast<unsigned *>(red + 8);
-    if (tid == 0) *last = __hip_atomic_fetch_add(arr, 1u, __ATOMIC_ACQ_REL, __HIP_MEMORY_SCOPE_AGENT);
-    __syncthreads();
+    if (tid == 0) *last = __hip_atomic_fetch_add(arr, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    lds_barrier();
     if (*last + 1 != (unsigned)P.nsplit) return;
-    __threadfence();
     const float *all = P.part + ((long long)n * P.heads + h) * P.nsplit * (dv + 2);
     auto rd = [&](int s, int i) { return __hip_atomic_load(all + (long long)s * (dv + 2) + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); };
+    // every wavefront: the splits' weights, a lane per split (sc: weights; a workgroup's splits fit it)
     float gm = -INFINITY;
-    for (int s = 0; s < P.nsplit; s++) gm = fmaxf(gm, rd(s, 0));
-    for (int d = tid; d < dv; d += 256) {
-        float a = 0.f, b = 0.f;
-        for (int s = 0; s < P.nsplit; s++) {
-            const float f = expf(rd(s, 0) - gm);
-            a += f * rd(s, 1);
-            b += f * rd(s, 2 + d);
+    for (int s = lane; s < P.nsplit; s += 64) gm = fmaxf(gm, rd(s, 0));
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) gm = fmaxf(gm, __shfl_xor(gm, o));
+    float den = 0.f;
+    for (int s = lane; s < P.nsplit; s += 64) {
+        const float m = rd(s, 0), f = m == -INFINITY ? 0.f : exp_f32(m - gm);
+        den += f * rd(s, 1);
+        if (w == 0) sc[s] = f;
+    }
+    den = wave_sum(den);
+    lds_barrier();
+    if (tid < dv) {
+        float a = 0.f;
+        for (int s0 = 0; s0 < P.nsplit; s0 += 8) {
+            float x[8];
+#pragma unroll
+            for (int i = 0; i < 8; i++) x[i] = rd(min(s0 + i, P.nsplit - 1), 2 + tid);
+#pragma unroll
+            for (int i = 0; i < 8; i++)
+                if (s0 + i < P.nsplit) a = fmaf(sc[s0 + i], x[i], a);
         }
-        finish(d, b / a);
+        finish(a / den);
     }
     if (tid == 0) __hip_atomic_store(arr, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
 }
 
 // a decode batch's mixers: grid (attention heads x splits + linear-attention heads, tokens)
-template <typename T>
+template <typename T, int M>
 __global__ void __launch_bounds__(256) mix_decode_kernel(WinParams A, GlaParams L) {
     extern __shared__ __align__(16) char lds[];
-    const int n = blockIdx.y, pos = A.pos[n], stream = A.stream[n], na = A.heads * A.nsplit;
-    if ((int)blockIdx.x < na) win_decode_block<T>(A, blockIdx.x / A.nsplit, blockIdx.x % A.nsplit, n, stream, pos, lds);
-    else gla_decode_block<T>(L, blockIdx.x - na, n, stream, pos, lds);
+    const int n = blockIdx.y, pos = A.pos[n], stream = A.stream[n], na = M ? A.heads * A.nsplit : 0;
+    if constexpr (M > 0) {
+        if ((int)blockIdx.x < na) {
+            win_decode_block<T, M>(A, blockIdx.x / A.nsplit, blockIdx.x % A.nsplit, n, stream, pos, lds);
+            return;
+        }
+    }
+    gla_decode_block<T>(L, blockIdx.x - na, n, stream, pos, lds);
 }
 
 template <typename T>
@@ -411,8 +444,14 @@ hipError_t launch_mix_decode(const WinParams &A, const GlaParams &L, int n, hipS
     size_t lds = 0;
     if (A.heads) lds = win_decode_lds(A.nks, A.nvt);
     if (L.heads) lds = std::max(lds, gla_decode_lds(L.dkp, L.dvp, L.rank));
-    hipLaunchKernelGGL(mix_decode_kernel<T>, dim3(A.heads * A.nsplit + L.heads, n), dim3(256), lds, st, A, L);
-    return hipGetLastError();
+    auto go = [&](auto kfn) {
+        hipLaunchKernelGGL(kfn, dim3(A.heads * A.nsplit + L.heads, n), dim3(256), lds, st, A, L);
+        return hipGetLastError();
+    };
+    if (!A.heads) return go(mix_decode_kernel<T, 0>);
+    if (A.nks <= 2) return go(mix_decode_kernel<T, 2>);
+    if (A.nks <= 4) return go(mix_decode_kernel<T, 4>);
+    return go(mix_decode_kernel<T, 8>);
 }
 
 template <typename T>

@@ -13,7 +13,7 @@ import sys
 
 import numpy as np
 
-MAX_STREAMS = 64
+MAX_STREAMS = 128
 
 
 def main(argv=None) -> int:
