@@ -678,7 +678,7 @@ def stack_sizes():
     return out
 
 
-def time_model(dev, vocab, streams, prompt_len=2047, pos=512, steps=128, batch_steps=32):
+def time_model(dev, vocab, streams, phases, prompt_len=2047, pos=512, steps=128, batch_steps=32):
     """Prompt, single-stream greedy decode and a batch of decode streams of one loaded model (host wall clock, best of three)."""
     import numpy as np
     from nanollama_amd import synth
@@ -697,9 +697,11 @@ def time_model(dev, vocab, streams, prompt_len=2047, pos=512, steps=128, batch_s
     def prompt():
         dev.reset()
         dev.prefill(toks)
-    prompt()
-    out = {"prompt_tokens": prompt_len, "prefill_ms": round(best(prompt) * 1e3, 3)}
-    out["prefill_tokens_per_s"] = round(prompt_len / out["prefill_ms"] * 1e3)
+    out = {}
+    if "prefill" in phases:
+        prompt()
+        out = {"prompt_tokens": prompt_len, "prefill_ms": round(best(prompt) * 1e3, 3)}
+        out["prefill_tokens_per_s"] = round(prompt_len / out["prefill_ms"] * 1e3)
 
     def chain():
         dev.reset()
@@ -709,26 +711,28 @@ def time_model(dev, vocab, streams, prompt_len=2047, pos=512, steps=128, batch_s
         for i in range(0, steps, 64):
             dev.decode_greedy(5, pos + i, 64)
         return time.perf_counter() - t0
-    chain()
-    dt = min(chain() for _ in range(3))
-    out.update(decode_position=pos, decode_ms=round(dt / steps * 1e3, 4), decode_tokens_per_s=round(steps / dt, 1))
-    ids = list(range(streams))
-    for s in ids:
-        dev.reset(s)
-        dev.prefill(toks[:64], 0, s, want_logits=False)
-    at = [64]
+    if "decode" in phases:
+        chain()
+        dt = min(chain() for _ in range(3))
+        out.update(decode_position=pos, decode_ms=round(dt / steps * 1e3, 4), decode_tokens_per_s=round(steps / dt, 1))
+    if "batch" in phases:
+        ids = list(range(streams))
+        for s in ids:
+            dev.reset(s)
+            dev.prefill(toks[:64], 0, s, want_logits=False)
+        at = [64]
 
-    def batch(n):
-        for _ in range(n):
-            dev.forward_batch(ids, [7 + s for s in ids], [at[0]] * streams)
-            at[0] += 1
-    batch(4)
-    dt = best(lambda: batch(batch_steps)) / batch_steps
-    out.update(batch_streams=streams, batch_ms_per_step=round(dt * 1e3, 4), batch_tokens_per_s=round(streams / dt))
+        def batch(n):
+            for _ in range(n):
+                dev.forward_batch(ids, [7 + s for s in ids], [at[0]] * streams)
+                at[0] += 1
+        batch(4)
+        dt = best(lambda: batch(batch_steps)) / batch_steps
+        out.update(batch_streams=streams, batch_ms_per_step=round(dt * 1e3, 4), batch_tokens_per_s=round(streams / dt))
     return out
 
 
-def stack_bench(names, only=None):
+def stack_bench(names, only=None, phases=("prefill", "decode", "batch")):
     """Ganidra (bfloat16) beside the quantised family's F16 files of equal size; random weights."""
     from nanollama_amd import _lib, gguf, model, synth_stack
     from nanollama_amd.designs import DESIGNS
@@ -741,13 +745,13 @@ def stack_bench(names, only=None):
             w = synth_stack.ganidra_weights(cfg, 1, fast=True)
             spec = DESIGNS["Ganidra"](cfg, lambda n: w[n].shape)
             dev = load_stack_model(spec, lambda n: ("BF16", w[n]), max_streams=64, seq_len=4096)
-            r["ganidra_bf16"] = dict(time_model(dev, shape.vocab, 64), params_millions=dev.config.num_params // 1000000)
+            r["ganidra_bf16"] = dict(time_model(dev, shape.vocab, 64, phases), params_millions=dev.config.num_params // 1000000)
             dev.close()
             del w
         if only != "ganidra":
             g = gguf.load_gguf(ensure_gguf(shape, "f16", "float"))
             dev = model.load_llama_model(g, max_streams=64)
-            r["llama_f16"] = dict(time_model(dev, shape.vocab, 64), params_millions=(shape.matrix_params() + shape.vocab * shape.dim) // 1000000)
+            r["llama_f16"] = dict(time_model(dev, shape.vocab, 64, phases), params_millions=(shape.matrix_params() + shape.vocab * shape.dim) // 1000000)
             dev.close()
         res[name] = r
         print(f"[bench] {name}: {json.dumps(r)}", file=sys.stderr, flush=True)
@@ -796,9 +800,10 @@ def main():
     ap.add_argument("--stack", nargs="?", const="mini,goldie,wide", default=None, metavar="SIZES",
                     help="one GPU: time the layer-stack design beside an F16 Llama of equal size and print that line only")
     ap.add_argument("--stack-only", choices=("ganidra", "llama"), default=None, help="with --stack: one of the two models")
+    ap.add_argument("--stack-phase", choices=("prefill", "decode", "batch"), default=None, help="with --stack: one of the three measurements (profiling)")
     args = ap.parse_args()
     if args.stack:
-        print(json.dumps(stack_bench(args.stack.split(","), args.stack_only)))
+        print(json.dumps(stack_bench(args.stack.split(","), args.stack_only, (args.stack_phase,) if args.stack_phase else ("prefill", "decode", "batch"))))
         return
     n = args.gpus
     if n < 1:
