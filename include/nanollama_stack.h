@@ -10,15 +10,22 @@
  * state is then zero whatever the stream held) or goes on where the stream's last call ended; anything else is NL_ERR_STATE.
  *
  * A layer is up to three residual branches' worth of description:
- *     x += mix_scale terms of { attention(norm1 x), linear_attention(norm1 x) }        (either may be absent)
- *     x += down(gelu_tanh(gate(norm2 x)) * up(norm2 x))                                (absent when ff == 0)
- * Norms are x / sqrt(mean(x^2) + eps) * (1 + w).  Tensor names for nl_upload_tensor (matrices [out, in]):
- *     embed                                    [vocab, dim]     token table; also the output matrix
+ *     x += mix_scale terms of { attention(norm1 x), linear_attention(norm1 x) }        (either may be absent), or
+ *     x += latent_attention(norm1 x)
+ *     x += down(act(gate(norm2 x)) * up(norm2 x))                                      (absent when ff == 0)
+ * With post_norm every sublayer's result goes through a norm of its own before it is added: x += norm1_post(mixer(norm1 x)), ....
+ * Norms are x / sqrt(mean(x^2) + eps) * (1 + w), or * w with plain_norm.  Tensor names for nl_upload_tensor (matrices [out, in]):
+ *     embed                                    [vocab, dim]     token table; also the output matrix unless untied
+ *     head                                     [vocab, dim]     output matrix (untied)
  *     final_norm                               [dim]
- *     layers.N.norm1 / norm2                   [dim]
+ *     layers.N.norm1 / norm2                   [dim]            and norm1_post / norm2_post with post_norm
  *     layers.N.attn.q / k / v / g / o          query, key, value, gate, output;  attn.q_norm / k_norm [head dim]
  *     layers.N.lin.q / k / v / g / o           likewise;  lin.a1 [rank, dim], lin.a2 [heads * dim, rank], lin.a2_bias, lin.norm [vdim]
- *     layers.N.ff.gate / up / down
+ *     layers.N.latent.dq / q_norm / uq         [q_rank, dim], [q_rank], [heads * (dim + rot_dim), q_rank]
+ *     layers.N.latent.dkv / kv_norm            [kv_rank + rot_dim, dim], [kv_rank]      (absent with kv_from)
+ *     layers.N.latent.uk / uv / o              [heads * dim, kv_rank], [heads * vdim, kv_rank], [dim, heads * vdim]
+ *     layers.N.latent.sink / g                 [heads], [heads, dim]
+ *     layers.N.ff.gate / up / down             and ff.gate_bias / up_bias / down_bias with ff_bias
  */
 #ifndef NANOLLAMA_STACK_H
 #define NANOLLAMA_STACK_H
@@ -49,10 +56,30 @@ typedef struct {
     float mix_scale;
 } nl_linattn_desc;
 
+/* latent attention: c_q = norm(dq h), [qu_h, qr_h] = uq c_q, [c, r] = dkv h with c normed, qr_h and r rotated by position;
+ * score_h = scale (qu_h . uk_h c + qr_h . r) over all earlier positions, values uv_h c; c and r are what is cached; heads == 0: none */
+typedef struct {
+    int32_t heads, dim, rot_dim, vdim;  /* per head: unrotated and rotated query-key size, value size */
+    int32_t q_rank, kv_rank;
+    int32_t kv_from;                    /* the earlier layer whose c and r (in its cache) this layer attends, -1: its own */
+    int32_t rot_dims;                   /* rotated dimensions of rot_dim (even), the rest pass */
+    int32_t rot_adjacent;               /* pairs are (2i, 2i + 1), else (i, i + rot_dims / 2) */
+    int32_t sink;                       /* a learned score per head in the softmax's denominator */
+    int32_t gate;                       /* head h's output *= sigmoid(g h)_h */
+    float scale;
+    double rope_base;
+    double yarn_factor, yarn_original, yarn_fast, yarn_slow;   /* YaRN interpolation; yarn_factor 0: none */
+} nl_latent_desc;
+
+enum { NL_ACT_GELU_TANH = 0, NL_ACT_SILU = 1 };
+
 typedef struct {
     nl_attn_desc attn;
     nl_linattn_desc lin;
-    int32_t ff; /* width of the gated feed-forward, 0: none */
+    nl_latent_desc latent; /* not beside attn or lin */
+    int32_t ff;            /* width of the gated feed-forward, 0: none */
+    int32_t ff_act;        /* NL_ACT_* */
+    int32_t ff_bias;       /* gate, up and down have biases */
 } nl_layer_desc;
 
 enum { NL_DTYPE_BF16 = 0, NL_DTYPE_F32 = 1 };
@@ -69,6 +96,9 @@ typedef struct {
     int32_t dtype;          /* NL_DTYPE_BF16: products and activations in bfloat16, 32-bit accumulation, everything else 32-bit;
                                NL_DTYPE_F32: 32-bit throughout */
     int32_t flags;          /* NL_FLAG_NO_GRAPH */
+    int32_t plain_norm;     /* norm gains are w instead of 1 + w */
+    int32_t post_norm;      /* a norm behind every sublayer (not with a loop) */
+    int32_t untied;         /* the output matrix is `head` */
     float eps, embed_scale;
 } nl_stack_config;
 
@@ -76,8 +106,9 @@ NL_API int nl_create_stack(const nl_stack_config *cfg, const nl_layer_desc *laye
 
 /* One ragged step: entry i brings n_tokens[i] tokens of stream streams[i] (distinct) from position pos0[i] on; `tokens` holds them one
  * entry behind the other.  want[0 .. n_want) are indices into `tokens` (ascending) whose logits are stored to logits_out
- * [n_want][vocab].  next_ids (may be NULL) [n_entries]: argmax behind each entry's last token.  Entries of one token each take the
- * decode launches, anything else the prompt launches; the result of a token does not depend on which. */
+ * [n_want][vocab].  next_ids (may be NULL) [n_entries]: argmax behind each entry's last token.  A step of one token per entry takes the
+ * decode launches, anything else the prompt launches; of a model with latent attention, one-token entries take the decode launches and
+ * the others the prompt launches.  The result of a token does not depend on which. */
 NL_API int nl_step(nl_handle h, int n_entries, const int *streams, const int *n_tokens, const int *pos0, const int *tokens,
                    int n_want, const int *want, float *logits_out, int *next_ids);
 /* Keep a copy of the residual stream behind every layer run of later calls (on != 0): nl_debug_read(h, "layers", 0, ...) returns

@@ -51,13 +51,19 @@ class NlLinattnDesc(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("heads", "dim", "vdim", "rank")] + [("tau", C.c_float), ("mix_scale", C.c_float)]
 
 
+class NlLatentDesc(C.Structure):
+    """nl_latent_desc: latent attention (heads == 0: none)."""
+    _fields_ = [(n, C.c_int32) for n in ("heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "kv_from", "rot_dims", "rot_adjacent", "sink", "gate")] + \
+               [("scale", C.c_float)] + [(n, C.c_double) for n in ("rope_base", "yarn_factor", "yarn_original", "yarn_fast", "yarn_slow")]
+
+
 class NlLayerDesc(C.Structure):
-    _fields_ = [("attn", NlAttnDesc), ("lin", NlLinattnDesc), ("ff", C.c_int32)]
+    _fields_ = [("attn", NlAttnDesc), ("lin", NlLinattnDesc), ("latent", NlLatentDesc)] + [(n, C.c_int32) for n in ("ff", "ff_act", "ff_bias")]
 
 
 class NlStackConfig(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("vocab", "dim", "n_layers", "loop_start", "loop_stop", "loop_times", "seq_len", "max_streams",
-                                         "max_step_tokens", "device", "dtype", "flags")] + \
+                                         "max_step_tokens", "device", "dtype", "flags", "plain_norm", "post_norm", "untied")] + \
                [("eps", C.c_float), ("embed_scale", C.c_float)]
 
 
@@ -67,8 +73,8 @@ class NlError(RuntimeError):
         self.code = code
 
 
-_STACK_ONLY = ("nl_linattn.h", "nl_mfma.h", "nl_winattn.h")
-_STACK_HEADERS = ("nl_kernels.h", "nl_linattn.h", "nl_mfma.h", "nl_sample.h", "nl_winattn.h")
+_STACK_ONLY = ("nl_latent.h", "nl_linattn.h", "nl_mfma.h", "nl_winattn.h")
+_STACK_HEADERS = ("nl_kernels.h", "nl_latent.h", "nl_linattn.h", "nl_mfma.h", "nl_sample.h", "nl_winattn.h")
 
 
 def source_files(family: str = "hip"):

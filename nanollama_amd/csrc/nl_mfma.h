@@ -13,8 +13,11 @@
 //
 // Two kernels: many_kernel for prompts (a 128 x 128 tile per workgroup, an LDS ring filled by LDS-DMA) and few_kernel for
 // decode batches of up to 64 tokens (one row tile per workgroup, K split over its wavefronts, the weights read once straight into
-// registers; for a handful of tokens the RMS norm of the layer's input runs in its prologue).  Epilogues: plain 32-bit store,
-// residual add (+ an optional second addend), gelu_tanh(gate) * up stored as the next product's operand.
+// registers; for a handful of tokens the RMS norm of the layer's input runs in its prologue, together with the norm and residual add
+// of the sublayer before where a model has norms behind its sublayers).  Epilogues: plain 32-bit store (+ bias), residual add (+ an
+// optional second addend), activation(gate) * up stored as the next product's operand, query rows by head with rotary positions, keys and
+// values in the operand order of the attention products.  A launch may carry independent work of single wavefronts behind its own
+// workgroups (TAIL).
 #pragma once
 #include "nl_kernels.h"
 
@@ -26,7 +29,7 @@ typedef bf16 bf16x4 __attribute__((ext_vector_type(4)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 constexpr int OPT = 512;          // elements of one operand tile (16 rows x 32 columns)
-enum { ST_F32 = 0, ST_RESID = 1, ST_GATED = 2 };   // epilogues
+enum { ST_F32 = 0, ST_RESID = 1, ST_GATED = 2, ST_HEADS = 3, ST_KEYS = 4, ST_VALUES = 5 };   // epilogues
 
 template <typename T> struct Frag;
 template <> struct Frag<bf16> { bf16x8 v; };
@@ -78,6 +81,7 @@ __device__ __forceinline__ float sigmoid_f32(float z) {
     const float e = exp_f32(-fminf(fabsf(z), 100.f)), r = rcp_f32(1.f + e);
     return z >= 0.f ? r : e * r;
 }
+__device__ __forceinline__ float silu_f32(float z) { return z * sigmoid_f32(z); }
 __device__ __forceinline__ float gelu_tanh_f32(float z) {
     // 0.5 (1 + tanh u) = sigmoid(2 u)
     return z * sigmoid_f32(1.5957691216057308f * (z + 0.044715f * z * z * z));
@@ -120,6 +124,19 @@ __global__ void pack_operand_kernel(const void *src, int src_f32, long long rows
         put(dst + op_index(((R >> 4) * tstride + toff) * 16 + (R & 15), k0 + c, nks), v);
     }
 }
+// the same with a place per source row: element (r, c) goes to row rbase[r], column kbase[r] + c, or transposed to row rbase[r] + c,
+// column kbase[r]
+template <typename T>
+__global__ void pack_mapped_kernel(const void *src, int src_f32, long long rows, long long cols, T *dst, int nks, const int *rbase, const int *kbase, int transpose) {
+    const long long n = rows * cols;
+    for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long long)gridDim.x * blockDim.x) {
+        const long long r = i / cols;
+        const int c = (int)(i - r * cols);
+        const float v = src_f32 ? reinterpret_cast<const float *>(src)[i]
+                                : __uint_as_float((unsigned)reinterpret_cast<const unsigned short *>(src)[i] << 16);
+        put(dst + op_index(rbase[r] + (transpose ? c : 0), kbase[r] + (transpose ? 0 : c), nks), v);
+    }
+}
 // a vector / small matrix as float, plus a constant (1 where a norm's gain is 1 + w); cols > 1: transposed to [cols][n / cols]
 __global__ void widen_kernel(const void *src, int src_f32, long long n, float add, float *dst, int cols) {
     for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long long)gridDim.x * blockDim.x)
@@ -146,52 +163,105 @@ __global__ void __launch_bounds__(256) lookup_kernel(LookupParams P) {
     }
 }
 
-// RMS norm of rows of the residual stream, stored as a product's operand (columns beyond dim zero)
+// work that rides in a launch: unit(i, lane) for i < units, one wavefront each, reading and writing nothing that the launch touches
+struct NoTail {
+    static constexpr bool on = false;
+    int units = 0;
+    __device__ __forceinline__ void unit(int, int) const {}
+};
+
+// RMS norm of rows of the residual stream, stored as a product's operand (columns beyond dim zero).  With d: the rows are first
+// x + norm(d) dw (a sublayer's result through the norm behind it), stored to x_out unless that is null.
 struct NormParams {
     const float *x, *w;    // w: the factor itself
     const int *rows;       // row of x for output token n; null: n
     void *out;
     int dim, nks, n_tokens;
     float eps;
+    int ld;                // floats between rows
+    const float *d, *dw;
+    float *x_out;
 };
-// grid (tiles of 16 tokens, splits of K): every workgroup sums the squares of its 16 rows and stores its share of the k tiles, whole
-// 16-row tiles at a time (contiguous stores)
-template <typename T>
-__global__ void __launch_bounds__(512) norm_operand_kernel(NormParams P) {
-    __shared__ float inv_s[16];
+// grid (tiles of 16 tokens, splits of K [+ 1 for the tail]): every workgroup sums the squares of its 16 rows and stores its share of the
+// k tiles, whole 16-row tiles at a time (contiguous stores)
+template <typename T, class TAIL>
+__global__ void __launch_bounds__(512) norm_operand_kernel(NormParams P, TAIL tail) {
+    __shared__ float inv_s[16], invd_s[16];
     const int n0 = blockIdx.x * 16, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+    const int nsplit = gridDim.y - (TAIL::on ? 1 : 0);
+    if constexpr (TAIL::on)
+        if ((int)blockIdx.y == nsplit) {
+            for (int i = 0; i < 2; i++)
+                if (n0 + w * 2 + i < tail.units) tail.unit(n0 + w * 2 + i, lane);
+            return;
+        }
     const bool vec = (P.dim & 3) == 0;
 #pragma unroll
     for (int i = 0; i < 2; i++) {
         const int n = min(n0 + w * 2 + i, P.n_tokens - 1);
-        const float *x = P.x + (long long)(P.rows ? P.rows[n] : n) * P.dim;
-        float ss = 0.f;
+        const long long at = (long long)(P.rows ? P.rows[n] : n) * P.ld;
+        const float *x = P.x + at, *d = P.d + at;
+        float ss = 0.f, invd = 0.f;
+        if (P.d) {
+            if (vec) {
+#pragma unroll 4
+                for (int k = lane * 4; k < P.dim; k += 256) {
+                    const f32x4 v = *reinterpret_cast<const f32x4 *>(d + k);
+                    ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+                }
+            } else
+                for (int k = lane; k < P.dim; k += 64) ss += d[k] * d[k];
+            invd = rsqrt_f32(wave_sum(ss) / (float)P.dim + P.eps);
+            if (lane == 0) invd_s[w * 2 + i] = invd;
+            ss = 0.f;
+        }
         if (vec) {
 #pragma unroll 4
             for (int k = lane * 4; k < P.dim; k += 256) {
-                const f32x4 v = *reinterpret_cast<const f32x4 *>(x + k);
+                f32x4 v = *reinterpret_cast<const f32x4 *>(x + k);
+                if (P.d) v += *reinterpret_cast<const f32x4 *>(d + k) * invd * *reinterpret_cast<const f32x4 *>(P.dw + k);
                 ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
             }
         } else
-            for (int k = lane; k < P.dim; k += 64) ss += x[k] * x[k];
+            for (int k = lane; k < P.dim; k += 64) {
+                const float v = P.d ? x[k] + d[k] * invd * P.dw[k] : x[k];
+                ss += v * v;
+            }
         ss = wave_sum(ss);
         if (lane == 0) inv_s[w * 2 + i] = rsqrt_f32(ss / (float)P.dim + P.eps);
     }
     __syncthreads();
     const int r = lane & 15, n = min(n0 + r, P.n_tokens - 1);
-    const float *x = P.x + (long long)(P.rows ? P.rows[n] : n) * P.dim;
-    const float inv = inv_s[r];
+    const long long at = (long long)(P.rows ? P.rows[n] : n) * P.ld;
+    const float *x = P.x + at, *d = P.d + at;
+    const float inv = inv_s[r], invd = P.d ? invd_s[r] : 0.f;
+    const bool keep = P.x_out && n0 + r < P.n_tokens;
     T *out = reinterpret_cast<T *>(P.out) + (long long)blockIdx.x * P.nks * OPT;
-    for (int ks = blockIdx.y * 8 + w; ks < P.nks; ks += gridDim.y * 8) {
+    for (int ks = blockIdx.y * 8 + w; ks < P.nks; ks += nsplit * 8) {
         const int k0 = ks * 32 + (lane >> 4) * 8;
         f32x4 a, b;
         if (vec && k0 + 8 <= P.dim) {
-            a = *reinterpret_cast<const f32x4 *>(x + k0) * inv * *reinterpret_cast<const f32x4 *>(P.w + k0);
-            b = *reinterpret_cast<const f32x4 *>(x + k0 + 4) * inv * *reinterpret_cast<const f32x4 *>(P.w + k0 + 4);
+            a = *reinterpret_cast<const f32x4 *>(x + k0);
+            b = *reinterpret_cast<const f32x4 *>(x + k0 + 4);
+            if (P.d) {
+                a += *reinterpret_cast<const f32x4 *>(d + k0) * invd * *reinterpret_cast<const f32x4 *>(P.dw + k0);
+                b += *reinterpret_cast<const f32x4 *>(d + k0 + 4) * invd * *reinterpret_cast<const f32x4 *>(P.dw + k0 + 4);
+            }
+            if (keep) {
+                *reinterpret_cast<f32x4 *>(P.x_out + at + k0) = a;
+                *reinterpret_cast<f32x4 *>(P.x_out + at + k0 + 4) = b;
+            }
+            a = a * inv * *reinterpret_cast<const f32x4 *>(P.w + k0);
+            b = b * inv * *reinterpret_cast<const f32x4 *>(P.w + k0 + 4);
         } else {
 #pragma unroll
             for (int j = 0; j < 8; j++) {
-                const float v = k0 + j < P.dim ? x[k0 + j] * inv * P.w[k0 + j] : 0.f;
+                float v = 0.f;
+                if (k0 + j < P.dim) {
+                    v = P.d ? x[k0 + j] + d[k0 + j] * invd * P.dw[k0 + j] : x[k0 + j];
+                    if (keep) P.x_out[at + k0 + j] = v;
+                    v *= inv * P.w[k0 + j];
+                }
                 if (j < 4) a[j] = v; else b[j - 4] = v;
             }
         }
@@ -200,14 +270,31 @@ __global__ void __launch_bounds__(512) norm_operand_kernel(NormParams P) {
         put4(o + 4, b);
     }
 }
-template <typename T>
-hipError_t launch_norm_operand(const NormParams &P, hipStream_t st) {
+template <typename T, class TAIL = NoTail>
+hipError_t launch_norm_operand(NormParams P, hipStream_t st, TAIL tail = {}) {
+    if (!P.ld) P.ld = P.dim;
     const int tt = (P.n_tokens + 15) / 16, split = std::max(1, std::min((P.nks + 7) / 8, 256 / tt));
-    hipLaunchKernelGGL(norm_operand_kernel<T>, dim3(tt, split), dim3(512), 0, st, P);
+    hipLaunchKernelGGL((norm_operand_kernel<T, TAIL>), dim3(tt, split + (TAIL::on ? 1 : 0)), dim3(512), 0, st, P, tail);
     return hipGetLastError();
 }
 
 // ----------------------------------------------------------- products ---
+
+// ST_HEADS: rows [0, split) are hrows[0] rows per head, the others hrows[1] rows per head; the latter's first `pairs` pairs of adjacent
+// rows are rotated by the token's position.  A row goes to q [token][head][ld] from column col[0 / 1] on, the first kind to the operand
+// xq (column = row) instead if there is one.
+struct HeadRows {
+    void *q, *xq;
+    int xq_nks, heads, ld, split, hrows[2], col[2], pairs;
+    const float *rope;     // [position][pairs] cos, sin
+    const int *pos;
+};
+// ST_KEYS / ST_VALUES: row = head * hrows + d, token = key slot; operand tiles [head][slots / 16][nt] (keys: nt tiles of 32 dimensions)
+// or [head][slots / 32][nt] (values: nt tiles of 16, the order of nl_winattn.h)
+struct KeyRows {
+    void *dst;
+    int hrows, nt, slots;
+};
 
 struct MatParams {
     const void *W;         // [nrt][nks] operand tiles; ST_GATED: gate tile, up tile, gate tile, ...
@@ -217,10 +304,17 @@ struct MatParams {
     int ldo;
     const float *add2;     // ST_RESID: also added (same layout as out), or null
     void *act;             // ST_GATED: [token tiles][act_nks] operand tiles
-    int act_nks;
-    // few_kernel with the norm in its prologue: B = norm(x)
-    const float *nx, *nw;
-    int ndim;
+    int act_nks, act_silu; // activation: silu or tanh-gelu
+    const float *bias, *bias2;   // ST_F32: per row; ST_GATED: of gate and up; whole row tiles long, or null
+    int x_nks;             // k tiles per token tile of X (0: nks)
+    int group;             // few_kernel: row tiles of a group; group i multiplies X's k tiles from i * nks on (0: one group)
+    const int *x_tile;     // many_kernel: which tile of X is token tile t (null: t)
+    HeadRows hd;
+    KeyRows kr;
+    // few_kernel with the norm in its prologue: B = norm(x), or of x + norm(nd) ndw, which workgroup 0 stores to nxo (may be null)
+    const float *nx, *nw, *nd, *ndw;
+    float *nxo;
+    int ndim, nld;         // nld: floats between rows (0: ndim)
     float neps;
     // one token: every row tile's largest result and its row, for the argmax that follows (or null)
     float *amax_val;
@@ -249,16 +343,47 @@ template <typename T>
 __device__ __forceinline__ void store_gated(const MatParams &P, int tok, int f16, int g, f32x4 gate, f32x4 up) {
     f32x4 v;
 #pragma unroll
-    for (int i = 0; i < 4; i++) v[i] = gelu_tanh_f32(gate[i]) * up[i];
+    for (int i = 0; i < 4; i++) {
+        if (P.bias) {
+            gate[i] += P.bias[f16 * 16 + 4 * g + i];
+            up[i] += P.bias2[f16 * 16 + 4 * g + i];
+        }
+        v[i] = (P.act_silu ? silu_f32(gate[i]) : gelu_tanh_f32(gate[i])) * up[i];
+    }
     put4(reinterpret_cast<T *>(P.act) + op_index(tok, f16 * 16 + 4 * g, P.act_nks), v);
+}
+
+__device__ __forceinline__ f32x4 with_bias(const float *bias, int row, f32x4 v) {
+    if (bias) v += *reinterpret_cast<const f32x4 *>(bias + row);
+    return v;
+}
+// four consecutive rows of one head of one token
+template <typename T>
+__device__ __forceinline__ void store_heads(const HeadRows &H, int tok, int row, f32x4 v) {
+    const int kind = row >= H.split, r0 = kind ? row - H.split : row, h = r0 / H.hrows[kind], d = r0 - h * H.hrows[kind];
+    if (h >= H.heads) return;
+    if (kind) {
+        const float *cs = H.rope + ((long long)H.pos[tok] * H.pairs + (d >> 1)) * 2;
+#pragma unroll
+        for (int i = 0; i < 2; i++)
+            if ((d >> 1) + i < H.pairs) {
+                const float c = cs[2 * i], s = cs[2 * i + 1], a = v[2 * i], b = v[2 * i + 1];
+                v[2 * i] = a * c - b * s;
+                v[2 * i + 1] = b * c + a * s;
+            }
+    } else if (H.xq) {
+        put4(reinterpret_cast<T *>(H.xq) + op_index(tok, row, H.xq_nks), v);
+        return;
+    }
+    put4(reinterpret_cast<T *>(H.q) + ((long long)tok * H.heads + h) * H.ld + H.col[kind] + d, v);
 }
 
 // prompts: RTW row tiles x 4 token tiles per wavefront, 2 x 2 wavefronts; the k tiles travel through a ring of LDS stages
 template <typename T, int RTW> struct ManyGeom {
     static constexpr int RT = 2 * RTW, NT = 8, UNIT = OPT * sizeof(T), NST = sizeof(T) == 2 ? 4 : 2, STAGE = (RT + NT) * UNIT, LDS = NST * STAGE;   // 48 or 64 KB
 };
-template <typename T, int EPI, int RTW>
-__global__ void __launch_bounds__(256) many_kernel(MatParams P) {
+template <typename T, int EPI, int RTW, class TAIL>
+__global__ void __launch_bounds__(256) many_kernel(MatParams P, TAIL tail) {
     using G = ManyGeom<T, RTW>;
     constexpr int RT = G::RT, NT = G::NT, UNIT = G::UNIT, NST = G::NST, STAGE = G::STAGE;
     constexpr int PW = STAGE / 4096;                       // 1 KiB pieces per stage and wavefront
@@ -267,7 +392,14 @@ __global__ void __launch_bounds__(256) many_kernel(MatParams P) {
     const int nrb = (P.nrt + RT - 1) / RT, ntt = (P.n_tokens + 15) >> 4, ntb = (ntt + NT - 1) / NT, total = nrb * ntb;
     // blocks b, b + 8, ... run on one XCD: give each XCD a contiguous range of (row block, token block), token blocks fastest, so
     // that the token blocks of a row block share its weights in one L2
-    const int per = (total + 7) / 8, id = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+    const int per = (total + 7) / 8;
+    if constexpr (TAIL::on)
+        if ((int)blockIdx.x >= per * 8) {
+            const int u = (blockIdx.x - per * 8) * 4 + w;
+            if (u < tail.units) tail.unit(u, lane);
+            return;
+        }
+    const int id = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
     if ((int)(blockIdx.x >> 3) >= per || id >= total) return;
     const int rb = id / ntb, tb = id - rb * ntb;
     const int wr = w & 1, wt = w >> 1, nks = P.nks;
@@ -276,8 +408,9 @@ __global__ void __launch_bounds__(256) many_kernel(MatParams P) {
 #pragma unroll
     for (int i = 0; i < PW; i++) {
         const int u = i * 4 + w, t = u / (UNIT / 1024), piece = u % (UNIT / 1024);
+        const int xt = min(tb * NT + t - RT, ntt - 1);
         src[i] = (t < RT ? reinterpret_cast<const char *>(P.W) + (long long)min(rb * RT + t, P.nrt - 1) * nks * UNIT
-                         : reinterpret_cast<const char *>(P.X) + (long long)min(tb * NT + t - RT, ntt - 1) * nks * UNIT) + piece * 1024 + lane * 16;
+                         : reinterpret_cast<const char *>(P.X) + (long long)(P.x_tile ? P.x_tile[xt] : xt) * P.x_nks * UNIT) + piece * 1024 + lane * 16;
     }
     auto issue = [&](int ks, int st) {
 #pragma unroll
@@ -301,8 +434,26 @@ __global__ void __launch_bounds__(256) many_kernel(MatParams P) {
         for (int r = 0; r < RTW; r++) {
             const Frag<T> a = *reinterpret_cast<const Frag<T> *>(base + (wr * RTW + r) * UNIT);
 #pragma unroll
-            for (int t = 0; t < 4; t++) acc[r][t] = mma(a, b[t], acc[r][t]);
+            for (int t = 0; t < 4; t++) acc[r][t] = EPI == ST_VALUES ? mma(b[t], a, acc[r][t]) : mma(a, b[t], acc[r][t]);
         }
+    }
+    if constexpr (EPI == ST_VALUES) {
+        // operands the other way round: a lane holds four consecutive keys of one value column, two token tiles are its fragment
+        const int tph = P.kr.hrows >> 4;
+#pragma unroll
+        for (int t = 0; t < 4; t += 2) {
+            const int kt = tb * NT + wt * 4 + t;
+            if (kt >= ntt) continue;
+#pragma unroll
+            for (int r = 0; r < RTW; r++) {
+                const int rt = rb * RT + wr * RTW + r, h = rt / tph;
+                if (rt >= P.nrt) continue;
+                T *o = reinterpret_cast<T *>(P.kr.dst) + ((((long long)h * (P.kr.slots >> 5) + (kt >> 1)) * P.kr.nt + rt - h * tph) * 64 + lane) * 8;
+                put4(o, acc[r][t]);
+                put4(o + 4, acc[r][t + 1]);
+            }
+        }
+        return;
     }
 #pragma unroll
     for (int t = 0; t < 4; t++) {
@@ -313,8 +464,12 @@ __global__ void __launch_bounds__(256) many_kernel(MatParams P) {
             const int rt = rb * RT + wr * RTW + r;
             if (rt >= P.nrt) continue;
             const int row = rt * 16 + 4 * g;
-            if constexpr (EPI == ST_F32) store_rows(P.out, P.ldo, P.rows, tok, row, acc[r][t]);
-            else if constexpr (EPI == ST_RESID) add_rows(P.out, P.add2, P.ldo, P.rows, tok, row, acc[r][t]);
+            if constexpr (EPI == ST_F32) store_rows(P.out, P.ldo, P.rows, tok, row, with_bias(P.bias, row, acc[r][t]));
+            else if constexpr (EPI == ST_HEADS) store_heads<T>(P.hd, tok, row, acc[r][t]);
+            else if constexpr (EPI == ST_KEYS) {
+                const int h = row / P.kr.hrows;
+                put4(reinterpret_cast<T *>(P.kr.dst) + (long long)h * P.kr.slots * P.kr.nt * 32 + op_index(tok, row - h * P.kr.hrows, P.kr.nt), acc[r][t]);
+            } else if constexpr (EPI == ST_RESID) add_rows(P.out, P.add2, P.ldo, P.rows, tok, row, acc[r][t]);
             else if constexpr (RTW > 1) {
                 if ((r & 1) == 0) store_gated<T>(P, tok, rt >> 1, g, acc[r][t], acc[r + (RTW > 1 ? 1 : 0)][t]);
             }
@@ -336,15 +491,22 @@ __device__ __forceinline__ void load_act(Frag<float> &f, const __amdgpu_buffer_r
 
 // decode batches: one row tile (ST_GATED: a gate and an up tile) x NT token tiles per workgroup, k tiles dealt to its WV wavefronts
 // in turn; a round's loads are all in flight together
-template <typename T, int EPI, int NT, int WV, bool NORM>
-__global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P) {
+// NORM: 0 none, 1 norm of nx, 2 norm of nx + norm(nd) ndw
+template <typename T, int EPI, int NT, int WV, int NORM, class TAIL>
+__global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P, TAIL tail) {
     constexpr int RB = EPI == ST_GATED ? 2 : 1;
     constexpr int PRE = (NT == 1 ? 8 : NT == 2 ? 6 : WV == 16 ? 4 : 6) / (sizeof(T) == 4 ? 2 : 1);
     extern __shared__ __align__(16) char lds[];
     const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, col = lane & 15;
     const int rt = blockIdx.x * RB, tt0 = blockIdx.y * NT, nks = P.nks, n = P.n_tokens;
+    if constexpr (TAIL::on)
+        if (rt >= P.nrt) {
+            const int u = (blockIdx.x - P.nrt / RB) * WV + w;
+            if (blockIdx.y == 0 && u < tail.units) tail.unit(u, lane);
+            return;
+        }
     // NORM: the residual rows are requested ahead of the weights (loads return in order)
-    float xv[NORM ? FEW_NORM_SLOTS : 1], wv[NORM ? FEW_NORM_SLOTS : 1];
+    float xv[NORM ? FEW_NORM_SLOTS : 1], wv[NORM ? FEW_NORM_SLOTS : 1], dv[NORM == 2 ? FEW_NORM_SLOTS : 1], dwv[NORM == 2 ? FEW_NORM_SLOTS : 1];
     const int ux = NORM ? (nks * 32 + 511) >> 9 : 1, nslots = NORM ? n * ux : 0;
     if constexpr (NORM) {
         int t = 0, u = 0;
@@ -352,13 +514,18 @@ __global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P) {
         for (int s = 0; s < FEW_NORM_SLOTS; s++)
             if (s < nslots) {
                 const int k = u * 512 + tid;
-                xv[s] = k < P.ndim ? P.nx[(long long)t * P.ndim + k] : 0.f;
+                if constexpr (NORM == 2) {
+                    dv[s] = k < P.ndim ? P.nd[(long long)t * P.nld + k] : 0.f;
+                    dwv[s] = k < P.ndim ? P.ndw[k] : 0.f;
+                }
+                xv[s] = k < P.ndim ? P.nx[(long long)t * P.nld + k] : 0.f;
                 wv[s] = k < P.ndim ? P.nw[k] : 0.f;
                 if (++u == ux) { u = 0; t++; }
             }
     }
     const Frag<T> *W = reinterpret_cast<const Frag<T> *>(P.W) + (long long)rt * nks * 64 + lane;
-    const __amdgpu_buffer_rsrc_t X = __builtin_amdgcn_make_buffer_rsrc(const_cast<void *>(P.X), 0, NORM ? 0 : (int)(((n + 15) >> 4) * nks * OPT * sizeof(T)), 0x00027000);
+    const __amdgpu_buffer_rsrc_t X = __builtin_amdgcn_make_buffer_rsrc(const_cast<void *>(P.X), 0, NORM ? 0 : (int)(((n + 15) >> 4) * P.x_nks * OPT * sizeof(T)), 0x00027000);
+    const int xk0 = P.group ? rt / P.group * nks : 0;
     f32x4 acc[RB][NT] = {};
     Frag<T> a[RB][PRE], b[PRE][NT];
     auto load = [&](int k0) {
@@ -371,7 +538,7 @@ __global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P) {
 #pragma unroll
                 for (int t = 0; t < NT; t++) {
                     frag_zero(b[u][t]);
-                    if ((tt0 + t) * 16 + col < n) load_act(b[u][t], X, (unsigned)((((tt0 + t) * nks + ks) * 64 + lane) * 8 * sizeof(T)));
+                    if ((tt0 + t) * 16 + col < n) load_act(b[u][t], X, (unsigned)((((tt0 + t) * P.x_nks + xk0 + ks) * 64 + lane) * 8 * sizeof(T)));
                 }
             }
         }
@@ -382,6 +549,38 @@ __global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P) {
         float *red = reinterpret_cast<float *>(lds + (size_t)nks * 32 * n * sizeof(T));      // [n][WV]
         int t = 0, u = 0;
         float ss = 0.f;
+        if constexpr (NORM == 2) {
+            float *redd = red + n * WV;
+#pragma unroll
+            for (int s = 0; s < FEW_NORM_SLOTS; s++)
+                if (s < nslots) {
+                    ss += dv[s] * dv[s];
+                    if (++u == ux) {
+                        ss = wave_sum(ss);
+                        if (lane == 0) redd[t * WV + w] = ss;
+                        ss = 0.f; u = 0; t++;
+                    }
+                }
+            lds_barrier();
+            const bool keep = P.nxo && blockIdx.x == 0 && blockIdx.y == 0;
+            float invd = 0.f;
+            t = u = 0;
+#pragma unroll
+            for (int s = 0; s < FEW_NORM_SLOTS; s++)
+                if (s < nslots) {
+                    if (u == 0) {
+                        float q = 0.f;
+#pragma unroll
+                        for (int i = 0; i < WV; i++) q += redd[t * WV + i];
+                        invd = rsqrt_f32(q / (float)P.ndim + P.neps);
+                    }
+                    xv[s] += dv[s] * invd * dwv[s];
+                    const int k = u * 512 + tid;
+                    if (keep && k < P.ndim) P.nxo[(long long)t * P.nld + k] = xv[s];
+                    if (++u == ux) { u = 0; t++; }
+                }
+            t = u = 0;
+        }
 #pragma unroll
         for (int s = 0; s < FEW_NORM_SLOTS; s++)
             if (s < nslots) {
@@ -456,57 +655,75 @@ __global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P) {
             if (l == 0) { P.amax_val[blockIdx.x] = best; P.amax_idx[blockIdx.x] = idx; }
         }
         if (tok >= n) continue;
-        if constexpr (EPI == ST_F32) store_rows(P.out, P.ldo, P.rows, tok, row, v[0]);
+        if constexpr (EPI == ST_F32) store_rows(P.out, P.ldo, P.rows, tok, row, with_bias(P.bias, row, v[0]));
+        else if constexpr (EPI == ST_HEADS) store_heads<T>(P.hd, tok, row, v[0]);
         else if constexpr (EPI == ST_RESID) add_rows(P.out, P.add2, P.ldo, P.rows, tok, row, v[0]);
         else store_gated<T>(P, tok, rt >> 1, l >> 4, v[0], v[RB - 1]);
     }
 }
 
-template <typename T, int EPI, int NT, int WV, bool NORM>
-hipError_t launch_few_nt(const MatParams &P, hipStream_t st) {
+template <typename T, int EPI, int NT, int WV, int NORM, class TAIL>
+hipError_t launch_few_nt(const MatParams &P, hipStream_t st, TAIL tail) {
     constexpr int RB = EPI == ST_GATED ? 2 : 1;
     const int tt = (P.n_tokens + 15) / 16;
     size_t lds = (size_t)WV * RB * NT * 64 * 16;           // at most 64 KB
-    if (NORM) lds = std::max(lds, (size_t)P.nks * 32 * P.n_tokens * sizeof(T) + (size_t)P.n_tokens * WV * 4);
-    hipLaunchKernelGGL((few_kernel<T, EPI, NT, WV, NORM>), dim3(P.nrt / RB, (tt + NT - 1) / NT), dim3(WV * 64), lds, st, P);
+    if (NORM) lds = std::max(lds, (size_t)P.nks * 32 * P.n_tokens * sizeof(T) + (size_t)P.n_tokens * WV * 4 * NORM);
+    hipLaunchKernelGGL((few_kernel<T, EPI, NT, WV, NORM, TAIL>), dim3(P.nrt / RB + (TAIL::on ? (tail.units + WV - 1) / WV : 0), (tt + NT - 1) / NT), dim3(WV * 64), lds, st, P, tail);
     return hipGetLastError();
 }
 // is the norm of the product's input computed inside the launch?
 inline bool few_norm_ok(int n, int nks) { return n * ((nks * 32 + 511) / 512) <= FEW_NORM_SLOTS; }
 
-template <typename T, int EPI>
-hipError_t launch_few(const MatParams &P, hipStream_t st, bool norm) {
+template <typename T, int EPI, class TAIL>
+hipError_t launch_few(const MatParams &P, hipStream_t st, int norm, TAIL tail) {
     constexpr int RB = EPI == ST_GATED ? 2 : 1;
-    if (norm) return launch_few_nt<T, EPI, 1, 8, true>(P, st);
+    if constexpr (EPI != ST_HEADS)
+        if (norm == 2) return launch_few_nt<T, EPI, 1, 8, 2>(P, st, tail);
+    if constexpr (EPI != ST_RESID)
+        if (norm) return launch_few_nt<T, EPI, 1, 8, 1>(P, st, tail);
     const int tt = (P.n_tokens + 15) / 16, blocks = P.nrt / RB;
     // few row tiles: sixteen wavefronts to a workgroup, and token tiles on workgroups of their own, until the chip is covered
     const bool deep = RB == 1 && blocks < 256 && P.nks >= 48;
     int nt = tt >= 3 ? 4 : tt;
     while (nt > 1 && blocks * ((tt + nt - 1) / nt) < 192) nt /= 2;
-    if constexpr (RB == 1) {
+    if constexpr (EPI == ST_HEADS) {
+        if (P.nks <= 8) {                                  // (a head's few k tiles)
+            if (nt == 1) return launch_few_nt<T, EPI, 1, 4, 0>(P, st, tail);
+            if (nt == 2) return launch_few_nt<T, EPI, 2, 4, 0>(P, st, tail);
+            return launch_few_nt<T, EPI, 4, 4, 0>(P, st, tail);
+        }
+    } else if constexpr (RB == 1) {
         if (deep) {
-            if (nt == 1) return launch_few_nt<T, EPI, 1, 16, false>(P, st);
-            if (nt == 2) return launch_few_nt<T, EPI, 2, 16, false>(P, st);
-            return launch_few_nt<T, EPI, 4, 16, false>(P, st);
+            if (nt == 1) return launch_few_nt<T, EPI, 1, 16, 0>(P, st, tail);
+            if (nt == 2) return launch_few_nt<T, EPI, 2, 16, 0>(P, st, tail);
+            return launch_few_nt<T, EPI, 4, 16, 0>(P, st, tail);
         }
     }
-    if (nt == 1) return launch_few_nt<T, EPI, 1, 8, false>(P, st);
-    if (nt == 2) return launch_few_nt<T, EPI, 2, 8, false>(P, st);
-    return launch_few_nt<T, EPI, 4, 8, false>(P, st);
+    if (nt == 1) return launch_few_nt<T, EPI, 1, 8, 0>(P, st, tail);
+    if (nt == 2) return launch_few_nt<T, EPI, 2, 8, 0>(P, st, tail);
+    return launch_few_nt<T, EPI, 4, 8, 0>(P, st, tail);
 }
 
-template <typename T, int EPI>
-hipError_t launch_product(MatParams P, hipStream_t st, bool norm = false) {
-    if (P.n_tokens <= 0) return hipSuccess;
-    if (P.n_tokens <= FEW_MAX_TOKENS) return launch_few<T, EPI>(P, st, norm);
+template <typename T, int EPI, class TAIL = NoTail>
+hipError_t launch_many(const MatParams &P, hipStream_t st, TAIL tail = {}) {
     const int ntb = (P.n_tokens + 127) / 128;
     auto go = [&](auto kfn, int rt, int lds) {
         const int total = (P.nrt + rt - 1) / rt * ntb;
-        hipLaunchKernelGGL(kfn, dim3((total + 7) / 8 * 8), dim3(256), lds, st, P);
+        hipLaunchKernelGGL(kfn, dim3((total + 7) / 8 * 8 + (TAIL::on ? (tail.units + 3) / 4 : 0)), dim3(256), lds, st, P, tail);
         return hipGetLastError();
     };
-    if ((P.nrt + 7) / 8 * ntb >= 512) return go(many_kernel<T, EPI, 4>, 8, ManyGeom<T, 4>::LDS);
-    return go(many_kernel<T, EPI, 2>, 4, ManyGeom<T, 2>::LDS);
+    if ((P.nrt + 7) / 8 * ntb >= 512) return go(many_kernel<T, EPI, 4, TAIL>, 8, ManyGeom<T, 4>::LDS);
+    return go(many_kernel<T, EPI, 2, TAIL>, 4, ManyGeom<T, 2>::LDS);
+}
+
+// norm: see few_kernel.  A tail rides in decode launches only (launch_few).
+template <typename T, int EPI, class TAIL = NoTail>
+hipError_t launch_product(MatParams P, hipStream_t st, int norm = 0, TAIL tail = {}) {
+    if (P.n_tokens <= 0) return hipSuccess;
+    if (!P.x_nks) P.x_nks = P.nks;
+    if (!P.nld) P.nld = P.ndim;
+    if (P.n_tokens <= FEW_MAX_TOKENS) return launch_few<T, EPI>(P, st, norm, tail);
+    return launch_many<T, EPI>(P, st);
 }
 
 }  // namespace nl

@@ -1,6 +1,6 @@
 // nl_winattn.h -- grouped-query softmax attention of the layer-stack models: optional per-head RMS norm of queries and keys, a
-// linear distance bias slope_h (i - j), an optional sliding window (keys i - window < j <= i), an output gate
-// sigmoid(g); query / key and value sizes may differ.  Scores, softmax and the norms are 32-bit; keys, values and the softmax
+// linear distance bias slope_h (i - j), an optional sliding window (keys i - window < j <= i), an optional learned score per head in
+// the denominator alone (prompts), an output gate sigmoid(g) per value or per head; query / key and value sizes may differ.  Scores, softmax and the norms are 32-bit; keys, values and the softmax
 // weights are operands of element type T (nl_mfma.h).
 //
 // CACHE.  A ring of R positions per (stream, kv head), position p in slot p % R, R a multiple of 64 and at least window - 1 + the
@@ -24,7 +24,8 @@ constexpr int WA_Q = 64;                  // queries per workgroup
 constexpr int WA_MAX_DIM = 256;
 constexpr int WA_SPLIT_KEYS = 2048;       // keys one split of the decode launch can hold
 
-struct WinTile { int tok0, nq, pos0, stream; };       // queries [tok0, tok0 + nq) of the step, first one at position pos0
+// queries [tok0, tok0 + nq) of the step, first one at position pos0; position p is in slot (key0 + p) % R
+struct WinTile { int tok0, nq, pos0, stream, key0; };
 
 struct WinParams {
     const float *proj;          // [token][ldp]
@@ -33,7 +34,8 @@ struct WinParams {
     int nks, nvt;               // key tiles of 32, value tiles of 16
     const float *qnorm, *knorm; // [dk] or null
     float eps, scale, oscale;
-    const float *slope;         // [heads]
+    const float *slope, *sink;  // [heads] or null
+    int head_gate;              // the gate is one value per head
     int window, R;              // window 0: everything
     void *K, *V;                // this layer run, stream 0
     long long kstride, vstride; // elements per stream
@@ -125,7 +127,7 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
     // queries of this wavefront: none of them sees keys outside [wlo, whi]
     const int wq = min(w * 16, tl.nq - 1), whi = tl.pos0 + min(w * 16 + 15, tl.nq - 1), wq0 = tl.pos0 + wq, wlo = max(0, wq0 - win + 1);
     auto issue = [&](int j, int st) {
-        const int slot = j % P.R;                        // R is a multiple of KT: a tile of keys is one contiguous run
+        const int slot = (tl.key0 + j) % P.R;            // R is a multiple of KT: a tile of keys is one contiguous run
         const char *ks = K + (long long)(slot >> 4) * nks * UNIT + lane * 16, *vs = V + (long long)(slot >> 5) * nvt * UNIT + lane * 16;
 #pragma unroll
         for (int i = 0; i < PW; i++) {                   // (the same number for every wavefront: pieces past the end repeat the last one)
@@ -208,9 +210,14 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
     l += __shfl_xor(l, 16);
     l += __shfl_xor(l, 32);
     if (qi >= tl.nq) return;
-    const float inv = P.oscale / l;
+    float inv = P.oscale / l;
+    if (P.sink) {
+        const float sk = P.sink[h] * LOG2E, mm = fmaxf(m, sk), f = exp2_f32(m - mm);
+        inv = P.oscale * f / (l * f + exp2_f32(sk - mm));
+    }
     T *y = reinterpret_cast<T *>(P.y);
-    const float *gz = P.proj + (long long)tok * P.ldp + P.off_g + h * P.dv;
+    const float *gz = P.proj + (long long)tok * P.ldp + P.off_g + (P.head_gate ? h : h * P.dv);
+    const int gs = P.head_gate ? 0 : 1;
 #pragma unroll
     for (int t = 0; t < 2 * M; t++)
         if (FULL || t < nvt) {
@@ -218,11 +225,11 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
             if (d + 3 < P.dv && (k & 3) == 0) {
                 f32x4 r;
 #pragma unroll
-                for (int i = 0; i < 4; i++) r[i] = o[t][i] * inv * (P.off_g < 0 ? 1.f : sigmoid_f32(gz[d + i]));
+                for (int i = 0; i < 4; i++) r[i] = o[t][i] * inv * (P.off_g < 0 ? 1.f : sigmoid_f32(gz[(d + i) * gs]));
                 put4(y + op_index(tok, k, P.y_nks), r);
             } else
                 for (int i = 0; i < 4; i++)
-                    if (d + i < P.dv) put(y + op_index(tok, k + i, P.y_nks), o[t][i] * inv * (P.off_g < 0 ? 1.f : sigmoid_f32(gz[d + i])));
+                    if (d + i < P.dv) put(y + op_index(tok, k + i, P.y_nks), o[t][i] * inv * (P.off_g < 0 ? 1.f : sigmoid_f32(gz[(d + i) * gs])));
         }
 }
 
@@ -455,8 +462,12 @@ hipError_t launch_mix_decode(const WinParams &A, const GlaParams &L, int n, hipS
 }
 
 template <typename T>
-hipError_t launch_win_attn(const WinParams &P, int n_tokens, int ntiles, hipStream_t st) {
+hipError_t launch_win_prep(const WinParams &P, int n_tokens, hipStream_t st) {
     hipLaunchKernelGGL(win_prep_kernel<T>, dim3(n_tokens, (P.heads + 2 * P.kv_heads + 3) / 4), dim3(256), 0, st, P);
+    return hipGetLastError();
+}
+template <typename T>
+hipError_t launch_win_attn(const WinParams &P, int ntiles, hipStream_t st) {
     const size_t stage = (size_t)((sizeof(T) == 2 ? 4 : 2) * P.nks + (sizeof(T) == 2 ? 2 : 1) * P.nvt) * OPT * sizeof(T);
     auto go = [&](auto kfn, int stages) {
         const size_t lds = stages * stage;

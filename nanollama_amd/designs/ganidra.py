@@ -44,4 +44,4 @@ def ganidra_spec(cfg: dict, shape: Callable[[str], Tuple[int, ...]]) -> StackSpe
         layers.append(layer)
     loop = cfg.get("loop")
     return StackSpec("Ganidra", cfg["vocab"], cfg["width"], layers, cfg["norm"]["eps"], cfg["embedding"]["scale"],
-                     (loop["start"], loop["stop"], loop["times"]) if loop else None, tensors)
+                     (loop["start"], loop["stop"], loop["times"]) if loop else None, tensors=tensors)

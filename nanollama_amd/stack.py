@@ -46,10 +46,47 @@ class LinearAttention:
 
 
 @dataclass
+class Yarn:
+    """Interpolated rotary frequencies."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass
+class LatentAttention:
+    """Softmax attention over keys and values that are images of one cached latent, see nl_latent_desc."""
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rope_base: float
+    rot_dims: int
+    adjacent_pairs: bool = False
+    yarn: Optional[Yarn] = None
+    kv_from: Optional[int] = None
+    sink: bool = False
+    gate: bool = False
+
+
+ACTIVATIONS = {"gelu_tanh": 0, "silu": 1}
+
+
+@dataclass
 class StackLayer:
     attn: Optional[Attention] = None
     lin: Optional[LinearAttention] = None
+    latent: Optional[LatentAttention] = None
     ff: int = 0
+    ff_act: str = "gelu_tanh"
+    ff_bias: bool = False
+
+    def mixers(self):
+        return [m for m in (self.attn, self.lin, self.latent) if m]
 
 
 @dataclass
@@ -61,6 +98,9 @@ class StackSpec:
     eps: float
     embed_scale: float = 1.0
     loop: Optional[Tuple[int, int, int]] = None      # start, stop, times
+    plain_norm: bool = False                         # norm gains are w, not 1 + w
+    post_norm: bool = False                          # a norm behind every sublayer
+    untied: bool = False                             # an output matrix of its own
     tensors: Dict[str, str] = field(default_factory=dict)   # library name -> name in the weight file
 
     def runs(self) -> List[int]:
@@ -79,7 +119,7 @@ class StackConfig:
         self.spec, self.seq_len, self.dtype, self.num_params = spec, seq_len, dtype, num_params
         self.architecture = spec.architecture
         self.num_layers, self.embed_dim, self.vocab_size = len(spec.layers), spec.dim, spec.vocab
-        self.num_heads = max(max(l.attn.heads if l.attn else 0, l.lin.heads if l.lin else 0) for l in spec.layers)
+        self.num_heads = max(m.heads for l in spec.layers for m in l.mixers())
         self.num_kv_heads = max((l.attn.kv_heads for l in spec.layers if l.attn), default=0)
         self.interm_size = max(l.ff for l in spec.layers)
         self.rms_norm_eps = spec.eps
@@ -128,7 +168,11 @@ def _layer_desc(layer: StackLayer) -> _lib.NlLayerDesc:
     if layer.lin:
         g = layer.lin
         d.lin = _lib.NlLinattnDesc(g.heads, g.dim, g.vdim, g.rank, g.tau, g.mix_scale)
-    d.ff = layer.ff
+    if layer.latent:
+        t, y = layer.latent, layer.latent.yarn or Yarn(0.0, 0.0, 0.0, 0.0)
+        d.latent = _lib.NlLatentDesc(t.heads, t.dim, t.rot_dim, t.vdim, t.q_rank, t.kv_rank, -1 if t.kv_from is None else t.kv_from, t.rot_dims,
+                                     int(t.adjacent_pairs), int(t.sink), int(t.gate), t.scale, t.rope_base, y.factor, y.original, y.fast, y.slow)
+    d.ff, d.ff_act, d.ff_bias = layer.ff, ACTIVATIONS[layer.ff_act], int(layer.ff_bias)
     return d
 
 
@@ -141,7 +185,7 @@ def load_stack_model(spec: StackSpec, get: Callable[[str], Tuple[str, np.ndarray
     seq_len = seq_len or DEFAULT_SEQ_LEN
     start, stop, times = spec.loop or (0, 0, 1)
     cfg = _lib.NlStackConfig(spec.vocab, spec.dim, len(spec.layers), start, stop, times, seq_len, max_streams, max_step_tokens, device,
-                             DTYPES[dtype], flags, spec.eps, spec.embed_scale)
+                             DTYPES[dtype], flags, int(spec.plain_norm), int(spec.post_norm), int(spec.untied), spec.eps, spec.embed_scale)
     descs = (_lib.NlLayerDesc * len(spec.layers))(*[_layer_desc(l) for l in spec.layers])
     h = C.c_void_p()
     rc = L.nl_create_stack(C.byref(cfg), descs, C.byref(h))

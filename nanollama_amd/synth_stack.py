@@ -53,6 +53,12 @@ def ganidra_shapes(cfg: dict, rank: int = 16) -> Dict[str, Tuple[int, ...]]:
     return out
 
 
+def _fast_matrix(rng, shape, size: float) -> np.ndarray:
+    n = shape[0] * shape[1]
+    bits = rng.integers(0, 1 << 63, size=(n + 3) // 4, dtype=np.int64).view(np.uint16)[:n].reshape(shape)
+    return (bits & np.uint16(0x807F)) | (np.uint16(127 + int(np.floor(np.log2(size)))) << np.uint16(7))
+
+
 def ganidra_weights(cfg: dict, seed: int, rank: int = 16, gain: float = 1.0, fast: bool = False) -> Dict[str, np.ndarray]:
     """bfloat16 bits by tensor name.  fast: matrices are +- a constant with random mantissas (benchmarks of large models)."""
     out = {}
@@ -65,13 +71,65 @@ def ganidra_weights(cfg: dict, seed: int, rank: int = 16, gain: float = 1.0, fas
         elif name.endswith("a2.b"):
             x = rng.uniform(-3.0, 5.0, shape)
         elif len(shape) == 2 and fast and not name.endswith(("a1", "a2")):
-            n = shape[0] * shape[1]
-            bits = rng.integers(0, 1 << 63, size=(n + 3) // 4, dtype=np.int64).view(np.uint16)[:n].reshape(shape)
-            expo = np.uint16(127 + int(np.floor(np.log2(gain / np.sqrt(shape[1] if name != "embed" else 1.0)))))
-            out[name] = (bits & np.uint16(0x807F)) | (expo << np.uint16(7))
+            out[name] = _fast_matrix(rng, shape, gain / np.sqrt(shape[1] if name != "embed" else 1.0))
             continue
         else:
             x = rng.standard_normal(shape) * (1.0 if name == "embed" else gain / np.sqrt(shape[1]))
+        out[name] = to_bf16(x.astype(np.float32))
+    return out
+
+
+def pabalix_layer(kind: int, ff: int = 0, **mixer) -> dict:
+    """kind 1, 2 or 3; mixer: heads, dim, rot_dim, vdim, kv_rank, q_rank, base, scale (default 1 / sqrt(dim + rot_dim)), yarn (factor,
+    original, fast, slow) or None, kv_from."""
+    m = {k: mixer[k] for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank")}
+    m["scale"] = mixer.get("scale") or (m["dim"] + m["rot_dim"]) ** -0.5
+    m["rot"] = {"base": float(mixer["base"]), "dims": m["rot_dim"]}
+    if mixer.get("yarn"):
+        m["rot"]["scaling"] = dict(zip(("factor", "original", "fast", "slow"), mixer["yarn"]))
+    if mixer.get("kv_from") is not None:
+        m["kv_from"] = mixer["kv_from"]
+    return {"type": "latent_attention" + ("" if kind == 1 else f"_{kind}"), "mixer": m, "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def pabalix_config(vocab: int, width: int, layers, eps: float = 1e-5) -> dict:
+    return {"architecture": "Pabalix", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": list(layers)}
+
+
+def pabalix_shapes(cfg: dict) -> Dict[str, Tuple[int, ...]]:
+    D = cfg["width"]
+    out: Dict[str, Tuple[int, ...]] = {"embed": (cfg["vocab"], D), "final.norm": (D,), "head": (cfg["vocab"], D)}
+    for i, L in enumerate(cfg["layers"]):
+        m, p = L["mixer"], f"l{i}.mix."
+        H, q, kv = m["heads"], m["q_rank"], m["kv_rank"]
+        out.update({f"l{i}.norm1": (D,), f"l{i}.norm1b": (D,), p + "dq": (q, D), p + "dq.norm": (q,), p + "uq": (H * (m["dim"] + m["rot_dim"]), q),
+                    p + "uk": (H * m["dim"], kv), p + "uv": (H * m["vdim"], kv), p + "o": (D, H * m["vdim"])})
+        if m.get("kv_from") is None:
+            out.update({p + "dkv": (kv + m["rot_dim"], D), p + "dkv.norm": (kv,)})
+        if L["type"].endswith("3"):
+            out.update({p + "sink": (H,), p + "g": (H, D)})
+        if L["mlp"]:
+            f, p = L["mlp"]["ff"], f"l{i}.mlp."
+            out.update({f"l{i}.norm2": (D,), f"l{i}.norm2b": (D,), p + "gate": (f, D), p + "gate.b": (f,), p + "up": (f, D), p + "up.b": (f,), p + "down": (D, f), p + "down.b": (D,)})
+    return out
+
+
+def pabalix_weights(cfg: dict, seed: int, gain: float = 1.0, fast: bool = False) -> Dict[str, np.ndarray]:
+    """bfloat16 bits by tensor name; fast as in ganidra_weights."""
+    out = {}
+    for name, shape in pabalix_shapes(cfg).items():
+        rng = np.random.Generator(np.random.PCG64([seed, zlib.crc32(name.encode())]))
+        if len(shape) == 2 and fast:
+            out[name] = _fast_matrix(rng, shape, 1.0 if name == "embed" else gain / np.sqrt(shape[1]))
+            continue
+        if len(shape) == 2:
+            x = rng.standard_normal(shape) * (1.0 if name == "embed" else gain / np.sqrt(shape[1]))
+        elif "norm" in name:
+            x = 1.0 + 0.2 * rng.standard_normal(shape)
+        elif name.endswith("sink"):
+            x = rng.uniform(-1.0, 3.0, shape)
+        else:
+            x = 0.3 * rng.standard_normal(shape)               # biases
         out[name] = to_bf16(x.astype(np.float32))
     return out
 

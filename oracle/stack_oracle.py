@@ -1,4 +1,4 @@
-"""Plain float64 restatement of the layer-stack models (Ganidra), one function per mechanism, whole sequences, no cache.
+"""Plain float64 restatement of the layer-stack models (Ganidra, Pabalix), one function per mechanism, whole sequences, no cache.
 
 TEST INFRASTRUCTURE ONLY -- importable from tests/, never from nanollama_amd/; it shares no code with the product.
 `cfg` is the dictionary of config.json, `w` a dictionary of float arrays by tensor name (matrices [out, in]).
@@ -113,8 +113,106 @@ def layer_runs(cfg):
     return runs + [(i, False) for i in range(b, n)]
 
 
+# ---- latent attention (Pabalix) -------------------------------------------------------------------------------------------------
+
+def norm_plain(x, weight, eps):
+    return rms(x, eps) * weight
+
+
+def rotary_frequencies(rot):
+    """(angle per position for each pair, factor of cos and sin); rot: dims, base and, for YaRN, scaling."""
+    n, base = rot["dims"], float(rot["base"])
+    f = base ** (-2.0 * np.arange(n // 2) / n)
+    y = rot.get("scaling")
+    if not y:
+        return f, 1.0
+    turns = lambda t: n * np.log(y["original"] / (2 * np.pi * t)) / (2 * np.log(base))    # the pair that turns t times over `original`
+    lo, hi = max(np.floor(turns(y["fast"])), 0.0), min(np.ceil(turns(y["slow"])), n - 1.0)
+    slow = np.clip((np.arange(n // 2) - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return f / y["factor"] * slow + f * (1.0 - slow), 0.1 * np.log(y["factor"]) + 1.0
+
+
+def rotate(x, rot, interleaved):
+    """x [T, ..., rot_dim], row t at position t."""
+    f, m = rotary_frequencies(rot)
+    a = np.arange(x.shape[0])[:, None] * f
+    shape = (x.shape[0],) + (1,) * (x.ndim - 2) + (len(f),)
+    c, s = (m * np.cos(a)).reshape(shape), (m * np.sin(a)).reshape(shape)
+    n = len(f)
+    first, second = (slice(0, 2 * n, 2), slice(1, 2 * n, 2)) if interleaved else (slice(0, n), slice(n, 2 * n))
+    out = x.copy()
+    out[..., first] = x[..., first] * c - x[..., second] * s
+    out[..., second] = x[..., second] * c + x[..., first] * s
+    return out
+
+
+def sink_softmax(s, sink=None):
+    """Rows of scores with -inf for unseen keys; sink: a score of the denominator alone."""
+    m = s.max(axis=-1, keepdims=True) if sink is None else np.maximum(s.max(axis=-1, keepdims=True), sink)
+    e = np.exp(s - m)
+    return e / (e.sum(axis=-1, keepdims=True) + (0.0 if sink is None else np.exp(sink - m)))
+
+
+LATENT_KINDS = {                 # type -> (adjacent dimensions are a pair, sink, gate per head)
+    "latent_attention": (False, False, False),
+    "latent_attention_2": (True, False, False),
+    "latent_attention_3": (False, True, True),
+}
+
+
+def latent_keys(h, m, w, p, eps, interleaved):
+    """(latent [T, kv_rank], rotated key part [T, rot_dim]): what a cache holds."""
+    c = h @ w[p + "dkv"].T
+    return norm_plain(c[:, :m["kv_rank"]], w[p + "dkv.norm"], eps), rotate(c[:, m["kv_rank"]:], m["rot"], interleaved)
+
+
+def latent_attention(h, m, w, p, eps, kind, held):
+    """held: latent_keys of this layer or of the layer that it borrows them from."""
+    H, d, r, v = m["heads"], m["dim"], m["rot_dim"], m["vdim"]
+    interleaved, sink, gate = LATENT_KINDS[kind]
+    T = h.shape[0]
+    q = (norm_plain(h @ w[p + "dq"].T, w[p + "dq.norm"], eps) @ w[p + "uq"].T).reshape(T, H, d + r)
+    qr = rotate(q[..., d:], m["rot"], interleaved)
+    c, kr = held
+    k = (c @ w[p + "uk"].T).reshape(T, H, d)
+    val = (c @ w[p + "uv"].T).reshape(T, H, v)
+    seen = np.tril(np.ones((T, T), bool))
+    out = np.zeros((T, H, v))
+    for a in range(H):
+        s = np.where(seen, (q[:, a, :d] @ k[:, a].T + qr[:, a] @ kr.T) * m["scale"], -np.inf)
+        out[:, a] = sink_softmax(s, w[p + "sink"][a] if sink else None) @ val[:, a]
+    if gate:
+        out = out * sigmoid(h @ w[p + "g"].T)[:, :, None]
+    return out.reshape(T, H * v) @ w[p + "o"].T
+
+
+def biased_silu_mlp(h, w, p):
+    return (silu(h @ w[p + "gate"].T + w[p + "gate.b"]) * (h @ w[p + "up"].T + w[p + "up.b"])) @ w[p + "down"].T + w[p + "down.b"]
+
+
+def latent_forward(cfg, w, tokens, want_layers=False):
+    """Pabalix: norms in front of and behind every sublayer, latent attention, an output matrix of its own."""
+    eps = cfg["norm"]["eps"]
+    x = w["embed"][np.asarray(tokens)]
+    seen, held = [], {}
+    for i, L in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", L["mixer"]
+        h = norm_plain(x, w[p + "norm1"], eps)
+        if m.get("kv_from") is None:
+            held[i] = latent_keys(h, m, w, p + "mix.", eps, LATENT_KINDS[L["type"]][0])
+        o = latent_attention(h, m, w, p + "mix.", eps, L["type"], held[i if m.get("kv_from") is None else m["kv_from"]])
+        x = x + norm_plain(o, w[p + "norm1b"], eps)
+        if L["mlp"] is not None:
+            x = x + norm_plain(biased_silu_mlp(norm_plain(x, w[p + "norm2"], eps), w, p + "mlp."), w[p + "norm2b"], eps)
+        seen.append(x)
+    logits = norm_plain(x, w["final.norm"], eps) @ w["head"].T
+    return (logits, np.stack(seen)) if want_layers else logits
+
+
 def forward(cfg, w, tokens, want_layers=False):
     """Logits [T, vocab] (and the residual stream after every layer run)."""
+    if cfg["architecture"] == "Pabalix":
+        return latent_forward(cfg, w, tokens, want_layers)
     eps = cfg["norm"]["eps"]
     x = w["embed"][np.asarray(tokens)] * cfg["embedding"]["scale"]
     x0 = x.copy()
