@@ -120,10 +120,10 @@ def pabalix_weights(cfg: dict, seed: int, gain: float = 1.0, fast: bool = False)
     for name, shape in pabalix_shapes(cfg).items():
         rng = np.random.Generator(np.random.PCG64([seed, zlib.crc32(name.encode())]))
         if len(shape) == 2 and fast:
-            out[name] = _fast_matrix(rng, shape, 1.0 if name == "embed" else gain / np.sqrt(shape[1]))
+            out[name] = _fast_matrix(rng, shape, 1.0 if name == "embed" else gain / np.sqrt(max(1, shape[1])))
             continue
         if len(shape) == 2:
-            x = rng.standard_normal(shape) * (1.0 if name == "embed" else gain / np.sqrt(shape[1]))
+            x = rng.standard_normal(shape) * (1.0 if name == "embed" else gain / np.sqrt(max(1, shape[1])))
         elif "norm" in name:
             x = 1.0 + 0.2 * rng.standard_normal(shape)
         elif name.endswith("sink"):

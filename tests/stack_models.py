@@ -22,8 +22,16 @@ def config(layers, vocab=96, width=64, loop=None, eps=1e-5, embed_scale=1.5):
     return ss.ganidra_config(vocab, width, layers, loop, eps, embed_scale)
 
 
+def lat(kind=1, heads=3, dim=16, rot=8, vdim=16, kv_rank=32, q_rank=24, base=500.0, scale=None, yarn=None, kv_from=None, ff=0):
+    return ss.pabalix_layer(kind, ff, heads=heads, dim=dim, rot_dim=rot, vdim=vdim, kv_rank=kv_rank, q_rank=q_rank, base=base, scale=scale, yarn=yarn, kv_from=kv_from)
+
+
+def lconfig(layers, vocab=96, width=64, eps=1e-5):
+    return ss.pabalix_config(vocab, width, layers, eps)
+
+
 def weights(cfg, seed=1, rank=4):
-    return ss.ganidra_weights(cfg, seed, rank)
+    return ss.pabalix_weights(cfg, seed) if cfg["architecture"] == "Pabalix" else ss.ganidra_weights(cfg, seed, rank)
 
 
 def floats(w):

@@ -18,7 +18,7 @@ from nanollama_amd.scheduler import Scheduler
 from nanollama_amd.synth_stack import write_folder
 from nanollama_amd.tokenizer import IdTokenizer
 from oracle import stack_oracle as so
-from stack_models import config, floats, gla, par, rel, tokens, weights
+from stack_models import F32_TOL, config, floats, gla, lat, lconfig, par, rel, tokens, weights
 
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
@@ -59,6 +59,12 @@ def test_create_fails_loudly_without_a_gpu_and_on_bad_shapes():
                       (config([gla()], loop=(0, 2, 2)), "loop range"), (config([par(window=-3)]), "attention sizes")):
         with pytest.raises(_lib.NlError, match=text):
             _create(bad, weights(bad))
+    for layers, text in (([lat(dim=250)], "up to 256"), ([lat(vdim=300)], "up to 256"), ([lat(kv_rank=760)], "up to 768"), ([lat(base=0.0)], "latent attention sizes"),
+                         ([lat(heads=0)], "no mixer"), ([lat(1, yarn=(-1.0, 9.0, 2.0, 1.0))], "rotary scaling"), ([lat(2), lat(2, kv_rank=40, kv_from=0)], "kv_from"),
+                         ([lat(2), lat(2, kv_from=1)], "kv_from"), ([lat(2), lat(2, kv_from=0), lat(2, kv_from=1)], "kv_from")):
+        bad = lconfig(layers)
+        with pytest.raises(_lib.NlError, match=text):
+            _create(bad, weights(bad))
     with pytest.raises(ValueError, match="dtype"):
         _create(cfg, w, dtype="float16")
 
@@ -83,6 +89,25 @@ def test_design_reads_every_size_and_constant():
     no_mask = copy.deepcopy(cfg)
     no_mask["layers"][1]["mixer"]["left"]["mask"] = None
     assert DESIGNS["Ganidra"](no_mask, lambda n: w[n].shape).layers[1].attn.window == 0
+
+
+def test_latent_design_reads_every_size_and_constant():
+    cfg = lconfig([lat(2, heads=3, dim=10, rot=6, vdim=7, kv_rank=13, q_rank=11, base=321.0, scale=0.37, ff=30), lat(1, heads=5, dim=12, rot=4, yarn=(1.5, 20.0, 4.0, 0.5)),
+                   lat(3, heads=2, kv_rank=9, yarn=(8.0, 640.0, 16.0, 2.0), ff=9), lat(2, heads=4, dim=8, rot=6, kv_rank=13, base=321.0, kv_from=0)], vocab=41, width=26, eps=3e-3)
+    w = weights(cfg)
+    s = DESIGNS["Pabalix"](cfg, lambda n: w[n].shape)
+    assert (s.vocab, s.dim, s.eps, s.embed_scale, s.loop, s.plain_norm, s.post_norm, s.untied) == (41, 26, 3e-3, 1.0, None, True, True, True)
+    a, b, c, d = (l.latent for l in s.layers)
+    assert (a.heads, a.dim, a.rot_dim, a.vdim, a.q_rank, a.kv_rank, a.scale, a.rope_base, a.rot_dims) == (3, 10, 6, 7, 11, 13, 0.37, 321.0, 6)
+    assert [(x.adjacent_pairs, x.sink, x.gate, x.kv_from) for x in (a, b, c, d)] == [(True, False, False, None), (False, False, False, None), (False, True, True, None), (True, False, False, 0)]
+    assert a.yarn is None and (b.yarn.factor, b.yarn.original, b.yarn.fast, b.yarn.slow) == (1.5, 20.0, 4.0, 0.5) and c.yarn.original == 640.0
+    assert [(l.ff, l.ff_bias) for l in s.layers] == [(30, True), (0, False), (9, True), (0, False)] and s.layers[0].ff_act == "silu"
+    assert sorted(s.tensors.values()) == sorted(w)         # every tensor of the file has exactly one place
+    for edit in (lambda x: x["layers"][0].update(type="latent_attention_9"), lambda x: x["layers"][0].update(mlp={"kind": "experts", "ff": 8})):
+        bad = copy.deepcopy(cfg)
+        edit(bad)
+        with pytest.raises(ValueError, match="unknown"):
+            DESIGNS["Pabalix"](bad, lambda n: w[n].shape)
 
 
 def test_unknown_designs_and_layers_are_refused(tmp_path):
@@ -271,3 +296,67 @@ def test_oracle_is_causal_and_loops_differ_from_repeated_layers():
     del again["loop"]
     w2 = dict(w, **{k.replace("l0.", "l2.", 1).replace("l1.", "l3.", 1): v for k, v in w.items() if k[:2] in ("l0", "l1")})
     assert rel(so.forward(again, w2, ids), full) > 1e-3      # (the passes of a loop start from x + the embedding)
+
+
+def test_oracle_rotation_depends_on_distance_alone():
+    rng = np.random.default_rng(2)
+    q, k = np.tile(rng.normal(size=10), (30, 1)), np.tile(rng.normal(size=10), (30, 1))
+    yarn = {"factor": 4.0, "original": 20.0, "fast": 8.0, "slow": 1.0}
+    for rot in ({"dims": 8, "base": 50.0}, {"dims": 8, "base": 50.0, "scaling": yarn}):
+        for adjacent in (False, True):
+            s = so.rotate(q, rot, adjacent) @ so.rotate(k, rot, adjacent).T
+            for d in range(29):
+                assert np.allclose(np.diagonal(s, -d), s[d, 0])
+            far = (1.0 if "scaling" not in rot else 0.1 * np.log(4.0) + 1.0) ** 2
+            assert np.allclose(s[0, 0], far * (q[0, :8] @ k[0, :8]) + q[0, 8:] @ k[0, 8:])
+
+
+def test_oracle_yarn_leaves_fast_pairs_and_stretches_slow_ones():
+    rot = {"dims": 64, "base": 10000.0}
+    f, one = so.rotary_frequencies(rot)
+    y, m = so.rotary_frequencies(dict(rot, scaling={"factor": 8.0, "original": 4096.0, "fast": 32.0, "slow": 1.0}))
+    turns = f * 4096.0 / (2 * np.pi)
+    assert one == 1.0 and np.isclose(m, 1.0 + 0.1 * np.log(8.0))
+    ratio = y / f
+    assert np.allclose(ratio[turns > 40], 1.0) and np.allclose(ratio[turns < 0.8], 1 / 8.0) and np.all(np.diff(ratio) <= 1e-12)
+    assert np.any((ratio < 0.9) & (ratio > 0.2))
+
+
+def test_oracle_sink_is_one_more_score_without_a_value():
+    rng = np.random.default_rng(3)
+    s = rng.normal(size=(4, 6))
+    s[0, 3:] = -np.inf
+    for sink in (-50.0, 0.3, 40.0):
+        e = np.exp(np.concatenate([s, np.full((4, 1), sink)], axis=1))
+        assert np.allclose(so.sink_softmax(s, sink), e[:, :6] / e.sum(axis=1, keepdims=True))
+    assert np.allclose(so.sink_softmax(s).sum(axis=-1), 1.0)
+
+
+def test_oracle_latent_model_is_causal_and_small_changes_of_a_constant_show():
+    """The mixed latent model has the power to show a fault: the oracle with one thing off is far outside the float32 tolerance."""
+    yarn = (4.0, 64.0, 8.0, 1.0)
+    cfg = lconfig([lat(2, rot=16, ff=16), lat(1, rot=16, yarn=yarn), lat(3, rot=16, yarn=yarn), lat(2, rot=16, kv_from=0)])
+    w, ids = floats(weights(cfg, 4)), tokens(60, seed=6)
+    full = so.forward(cfg, w, ids)
+    assert rel(so.forward(cfg, w, ids[:23]), full[:23]) < 1e-12
+
+    def off(edit):
+        c = copy.deepcopy(cfg)
+        edit(c["layers"])
+        return rel(so.forward(c, w, ids), full)
+    mix = lambda i, **kw: (lambda L: L[i]["mixer"].update(kw))
+    rot = lambda i, **kw: (lambda L: L[i]["mixer"]["rot"].update(kw))
+    scl = lambda i, **kw: (lambda L: L[i]["mixer"]["rot"]["scaling"].update(kw))
+    kind = lambda i, t: (lambda L: L[i].update(type=t))
+    edits = [mix(0, scale=0.21), rot(0, base=510.0), kind(0, "latent_attention"), kind(1, "latent_attention_2"), kind(2, "latent_attention"), scl(1, factor=4.2), scl(1, original=80.0),
+             scl(2, fast=3.0), scl(2, slow=5.0), lambda L: L[1]["mixer"]["rot"].pop("scaling"), lambda L: L[0].update(mlp=None)]
+    for n, e in enumerate(edits):
+        assert off(e) > 20 * F32_TOL, n
+    for name in ("l0.norm1b", "l3.norm1b", "l0.norm2b", "l2.mix.sink", "l0.mlp.gate.b", "l0.mlp.up.b", "l0.mlp.down.b", "l1.mix.dq.norm", "l1.mix.dkv.norm"):
+        w2 = dict(w)
+        w2[name] = w[name] + 0.1
+        assert rel(so.forward(cfg, w2, ids), full) > 20 * F32_TOL, name
+    own = copy.deepcopy(cfg)
+    del own["layers"][3]["mixer"]["kv_from"]
+    w2 = dict(w, **{"l3.mix.dkv": w["l0.mix.dkv"], "l3.mix.dkv.norm": w["l0.mix.dkv.norm"]})
+    assert rel(so.forward(own, w2, ids), full) > 20 * F32_TOL     # (the latents are layer 0's, not layer 0's matrix on layer 3's input)
