@@ -662,14 +662,22 @@ def shard_probe(model, rdv, ns=(2, 4, 8), seam_us=2.0, steps=96, warmup=16, base
 
 # ------------------------------------------------------------------ layer-stack models (--stack) ---
 
-def stack_sizes():
-    """name -> (Llama shape, Ganidra configuration) of equal width, depth, feed-forward and vocabulary.  Every fourth Ganidra layer is
-    a parallel one (softmax attention over a 1024-token window beside linear attention), the others are linear attention."""
+def stack_sizes(design="ganidra"):
+    """name -> (Llama shape, configuration) of equal width, depth, feed-forward and vocabulary.  Ganidra: every fourth layer is a parallel
+    one (softmax attention over a 1024-token window beside linear attention), the others are linear attention.  Pabalix: the three kinds of
+    latent attention in turn, D / 128 heads, latents of 256 (width 4096: 512) beside 64 rotated dimensions, every fourth layer attends the
+    latents of the one two before it."""
     from nanollama_amd import synth
-    from nanollama_amd.synth_stack import ganidra_config, ganidra_layer
+    from nanollama_amd.synth_stack import ganidra_config, ganidra_layer, pabalix_config, pabalix_layer
     out = {}
     for name, L, D, V in (("mini", 20, 768, 32000), ("goldie", 28, 1536, 48000), ("wide", 4, 4096, 32000)):
         shape = synth.ModelShape("stackbench_" + name, L, D, D // 64, D // 256, V)
+        if design == "pabalix":
+            size = dict(heads=D // 128, dim=128, rot_dim=64, vdim=128, kv_rank=512 if D >= 4096 else 256, q_rank=D // 2, base=10000.0)
+            yarn = (4.0, 4096.0, 32.0, 1.0)
+            kinds = [pabalix_layer(1, shape.ffn, yarn=yarn, **size), pabalix_layer(2, shape.ffn, **size), pabalix_layer(3, shape.ffn, yarn=yarn, **size)]
+            out[name] = (shape, pabalix_config(V, D, [kinds[i % 4] if i % 4 < 3 else pabalix_layer(2, shape.ffn, kv_from=i - 2, **size) for i in range(L)]))
+            continue
         lin = lambda h: dict(heads=h, dim=64, vdim=128, tau=16.0)
         par = ganidra_layer("parallel", shape.ffn, left=dict(heads=D // 128, kv_heads=max(1, D // 512), dim=64, vdim=64, scale=0.125, mask={"size": 1024}),
                             left_scale=0.7, right=lin(D // 256), right_scale=0.7)
@@ -732,31 +740,31 @@ def time_model(dev, vocab, streams, phases, prompt_len=2047, pos=512, steps=128,
     return out
 
 
-def stack_bench(names, only=None, phases=("prefill", "decode", "batch")):
-    """Ganidra (bfloat16) beside the quantised family's F16 files of equal size; random weights."""
+def stack_bench(names, only=None, phases=("prefill", "decode", "batch"), design="ganidra"):
+    """A layer-stack design (bfloat16) beside the quantised family's F16 files of equal size; random weights."""
     from nanollama_amd import _lib, gguf, model, synth_stack
     from nanollama_amd.designs import DESIGNS
     from nanollama_amd.stack import load_stack_model
     res = {}
     for name in names:
-        shape, cfg = stack_sizes()[name]
+        shape, cfg = stack_sizes(design)[name]
         r = {}
         if only != "llama":
-            w = synth_stack.ganidra_weights(cfg, 1, fast=True)
-            spec = DESIGNS["Ganidra"](cfg, lambda n: w[n].shape)
+            w = (synth_stack.pabalix_weights if design == "pabalix" else synth_stack.ganidra_weights)(cfg, 1, fast=True)
+            spec = DESIGNS[cfg["architecture"]](cfg, lambda n: w[n].shape)
             dev = load_stack_model(spec, lambda n: ("BF16", w[n]), max_streams=64, seq_len=4096)
-            r["ganidra_bf16"] = dict(time_model(dev, shape.vocab, 64, phases), params_millions=dev.config.num_params // 1000000)
+            r[design + "_bf16"] = dict(time_model(dev, shape.vocab, 64, phases), params_millions=dev.config.num_params // 1000000)
             dev.close()
             del w
-        if only != "ganidra":
+        if only in (None, "llama"):
             g = gguf.load_gguf(ensure_gguf(shape, "f16", "float"))
             dev = model.load_llama_model(g, max_streams=64)
             r["llama_f16"] = dict(time_model(dev, shape.vocab, 64, phases), params_millions=(shape.matrix_params() + shape.vocab * shape.dim) // 1000000)
             dev.close()
         res[name] = r
         print(f"[bench] {name}: {json.dumps(r)}", file=sys.stderr, flush=True)
-    return {"metric": "layer-stack model (Ganidra) and F16 Llama of equal size: prefill / decode / 64-stream decode", "unit": "tokens/s",
-            "value": res[names[-1]].get("ganidra_bf16", {}).get("decode_tokens_per_s"), "n_gpus": 1, "higher_is_better": True, "vs_baseline": None,
+    return {"metric": f"layer-stack model ({design.capitalize()}) and F16 Llama of equal size: prefill / decode / 64-stream decode", "unit": "tokens/s",
+            "value": res[names[-1]].get(design + "_bf16", {}).get("decode_tokens_per_s"), "n_gpus": 1, "higher_is_better": True, "vs_baseline": None,
             "dtype": "bf16", "data": "synthetic (random weights)", "sizes": res, "lib": _lib.source_sha(_lib.source_files("stack"))}
 
 
@@ -799,11 +807,12 @@ def main():
     ap.add_argument("--profile-pos", type=int, default=None, help="position of the per-launch profile (default: the mean timed position)")
     ap.add_argument("--stack", nargs="?", const="mini,goldie,wide", default=None, metavar="SIZES",
                     help="one GPU: time the layer-stack design beside an F16 Llama of equal size and print that line only")
-    ap.add_argument("--stack-only", choices=("ganidra", "llama"), default=None, help="with --stack: one of the two models")
+    ap.add_argument("--stack-design", choices=("ganidra", "pabalix"), default="ganidra", help="with --stack: which layer-stack design")
+    ap.add_argument("--stack-only", choices=("stack", "llama"), default=None, help="with --stack: one of the two models")
     ap.add_argument("--stack-phase", choices=("prefill", "decode", "batch"), default=None, help="with --stack: one of the three measurements (profiling)")
     args = ap.parse_args()
     if args.stack:
-        print(json.dumps(stack_bench(args.stack.split(","), args.stack_only, (args.stack_phase,) if args.stack_phase else ("prefill", "decode", "batch"))))
+        print(json.dumps(stack_bench(args.stack.split(","), args.stack_only, (args.stack_phase,) if args.stack_phase else ("prefill", "decode", "batch"), args.stack_design)))
         return
     n = args.gpus
     if n < 1:

@@ -86,10 +86,14 @@ __device__ __forceinline__ float gelu_tanh_f32(float z) {
     // 0.5 (1 + tanh u) = sigmoid(2 u)
     return z * sigmoid_f32(1.5957691216057308f * (z + 0.044715f * z * z * z));
 }
+template <int CTRL> __device__ __forceinline__ float dpp_add(float v) {
+    return v + __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
+}
+__device__ __forceinline__ float lane_value(float v, int lane) { return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), lane)); }
+// sum over the wavefront, in every lane: rows of 16 lanes by DPP (neighbours, pairs, mirrored halves, mirrored row), then the four rows
 __device__ __forceinline__ float wave_sum(float v) {
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
-    return v;
+    v = dpp_add<0x140>(dpp_add<0x141>(dpp_add<0x4E>(dpp_add<0xB1>(v))));
+    return (lane_value(v, 0) + lane_value(v, 16)) + (lane_value(v, 32) + lane_value(v, 48));
 }
 
 // 16 bytes per lane straight into LDS: lane i lands at lds_base + 16 i (lds_base wave-uniform)
@@ -270,9 +274,109 @@ __global__ void __launch_bounds__(512) norm_operand_kernel(NormParams P, TAIL ta
         put4(o + 4, b);
     }
 }
+// the same for rows that fit a workgroup's registers, read once: RW rows per workgroup, a thread holds NU runs of 8 columns of one row.
+// RW 1 spreads a decode batch over the chip; RW 8 stores whole 128-byte lines of the operand.  [+ workgroups for the tail]
+template <typename T, int RW, int NU, int NTHR, class TAIL>
+__global__ void __launch_bounds__(NTHR) norm_rows_kernel(NormParams P, TAIL tail) {
+    constexpr int NW = NTHR / 64;
+    __shared__ float red[2][NW][RW];
+    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, nb = (P.n_tokens + RW - 1) / RW;
+    if constexpr (TAIL::on)
+        if ((int)blockIdx.x >= nb) {
+            const int u = (blockIdx.x - nb) * NW + w;
+            if (u < tail.units) tail.unit(u, lane);
+            return;
+        }
+    const int r = tid % RW, n = blockIdx.x * RW + r, row = min(n, P.n_tokens - 1), runs = P.nks * 4;
+    const long long at = (long long)(P.rows ? P.rows[row] : row) * P.ld;
+    f32x4 v[NU][2] = {}, d[NU][2] = {}, wv[NU][2] = {};
+    auto each = [&](auto f) {                              // (run, columns of it that exist)
+#pragma unroll
+        for (int i = 0; i < NU; i++) {
+            const int run = tid / RW + i * (NTHR / RW);
+            if (run < runs) f(i, run * 8, P.dim - run * 8);
+        }
+    };
+    auto read = [&](f32x4 *o, const float *p, int k0, int left) {
+        if (left >= 8 && (P.dim & 3) == 0) {
+            o[0] = *reinterpret_cast<const f32x4 *>(p + k0);
+            o[1] = *reinterpret_cast<const f32x4 *>(p + k0 + 4);
+        } else
+#pragma unroll
+            for (int j = 0; j < 8; j++)
+                if (j < left) o[j >> 2][j & 3] = p[k0 + j];
+    };
+    // sum of squares of the thread's values over its row
+    auto row_sum = [&](f32x4 (&x)[NU][2], int k) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < NU; i++)
+#pragma unroll
+            for (int j = 0; j < 8; j++) ss += x[i][j >> 2][j & 3] * x[i][j >> 2][j & 3];
+        if constexpr (RW == 1) ss = wave_sum(ss);
+        else
+#pragma unroll
+            for (int o = RW; o < 64; o <<= 1) ss += __shfl_xor(ss, o);
+        if (lane < RW) red[k][w][lane] = ss;
+        lds_barrier();
+        ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < NW; i++) ss += red[k][i][r];
+        return rsqrt_f32(ss / (float)P.dim + P.eps);
+    };
+    each([&](int i, int k0, int left) {
+        if (P.d) read(d[i], P.d + at, k0, left);
+        read(v[i], P.x + at, k0, left);
+    });
+    f32x4 dw[NU][2] = {};
+    each([&](int i, int k0, int left) {
+        if (P.d) read(dw[i], P.dw, k0, left);
+        read(wv[i], P.w, k0, left);
+    });
+    if (P.d) {
+        const float inv = row_sum(d, 0);
+        each([&](int i, int k0, int left) {
+#pragma unroll
+            for (int h = 0; h < 2; h++) v[i][h] += d[i][h] * inv * dw[i][h];
+            if (!P.x_out || n >= P.n_tokens) return;
+            float *o = P.x_out + at + k0;
+            if (left >= 8 && (P.dim & 3) == 0) {
+                *reinterpret_cast<f32x4 *>(o) = v[i][0];
+                *reinterpret_cast<f32x4 *>(o + 4) = v[i][1];
+            } else
+#pragma unroll
+                for (int j = 0; j < 8; j++)
+                    if (j < left) o[j] = v[i][j >> 2][j & 3];
+        });
+    }
+    const float inv = row_sum(v, 1);
+    if (n >= P.n_tokens) return;
+    each([&](int i, int k0, int) {
+        T *o = reinterpret_cast<T *>(P.out) + op_index(n, k0, P.nks);
+        put4(o, v[i][0] * inv * wv[i][0]);
+        put4(o + 4, v[i][1] * inv * wv[i][1]);
+    });
+}
+constexpr int NORM_FEW_ROWS = 256;        // rows up to which every row has a workgroup of its own
+
 template <typename T, class TAIL = NoTail>
 hipError_t launch_norm_operand(NormParams P, hipStream_t st, TAIL tail = {}) {
     if (!P.ld) P.ld = P.dim;
+    if ((P.ld & 3) == 0 || (P.dim & 3)) {                  // (rows of vectors start at vectors)
+        const int runs = P.nks * 4;
+        auto go = [&](auto kfn, int rw, int nthr) {
+            hipLaunchKernelGGL(kfn, dim3((P.n_tokens + rw - 1) / rw + (TAIL::on ? (tail.units + nthr / 64 - 1) / (nthr / 64) : 0)), dim3(nthr), 0, st, P, tail);
+            return hipGetLastError();
+        };
+        if (P.n_tokens <= NORM_FEW_ROWS) {
+            if (runs <= 256) return go(norm_rows_kernel<T, 1, 1, 256, TAIL>, 1, 256);
+            if (runs <= 1024) return go(norm_rows_kernel<T, 1, 4, 256, TAIL>, 1, 256);
+        } else {
+            if (runs <= 128) return go(norm_rows_kernel<T, 8, 1, 1024, TAIL>, 8, 1024);
+            if (runs <= 256) return go(norm_rows_kernel<T, 8, 2, 1024, TAIL>, 8, 1024);
+            if (runs <= 512) return go(norm_rows_kernel<T, 4, 2, 1024, TAIL>, 4, 1024);
+        }
+    }
     const int tt = (P.n_tokens + 15) / 16, split = std::max(1, std::min((P.nks + 7) / 8, 256 / tt));
     hipLaunchKernelGGL((norm_operand_kernel<T, TAIL>), dim3(tt, split + (TAIL::on ? 1 : 0)), dim3(512), 0, st, P, tail);
     return hipGetLastError();
@@ -478,7 +582,7 @@ __global__ void __launch_bounds__(256) many_kernel(MatParams P, TAIL tail) {
 }
 
 constexpr int FEW_MAX_TOKENS = 64;
-constexpr int FEW_NORM_SLOTS = 16;        // (token, 512 columns) slots up to which few_kernel computes the norm itself
+constexpr int FEW_NORM_SLOTS = 4;         // (token, 2048 columns) slots up to which few_kernel computes the norm itself
 
 // activations go round the vector L1 (sc1): they are L2-resident and every workgroup streams them once
 __device__ __forceinline__ void load_act(Frag<bf16> &f, const __amdgpu_buffer_rsrc_t rs, unsigned byte_off) {
@@ -491,8 +595,9 @@ __device__ __forceinline__ void load_act(Frag<float> &f, const __amdgpu_buffer_r
 
 // decode batches: one row tile (ST_GATED: a gate and an up tile) x NT token tiles per workgroup, k tiles dealt to its WV wavefronts
 // in turn; a round's loads are all in flight together
-// NORM: 0 none, 1 norm of nx, 2 norm of nx + norm(nd) ndw
-template <typename T, int EPI, int NT, int WV, int NORM, class TAIL>
+// NORM: 0 none, 1 norm of nx, 2 norm of nx + norm(nd) ndw; NS: bound of its (token, 2048 columns) slots, four columns per thread and slot
+// (kept small: a launch this short is held up by fetching its own instructions)
+template <typename T, int EPI, int NT, int WV, int NORM, int NS, class TAIL>
 __global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P, TAIL tail) {
     constexpr int RB = EPI == ST_GATED ? 2 : 1;
     constexpr int PRE = (NT == 1 ? 8 : NT == 2 ? 6 : WV == 16 ? 4 : 6) / (sizeof(T) == 4 ? 2 : 1);
@@ -506,20 +611,22 @@ __global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P, TAIL tail) {
             return;
         }
     // NORM: the residual rows are requested ahead of the weights (loads return in order)
-    float xv[NORM ? FEW_NORM_SLOTS : 1], wv[NORM ? FEW_NORM_SLOTS : 1], dv[NORM == 2 ? FEW_NORM_SLOTS : 1], dwv[NORM == 2 ? FEW_NORM_SLOTS : 1];
-    const int ux = NORM ? (nks * 32 + 511) >> 9 : 1, nslots = NORM ? n * ux : 0;
+    f32x4 xv[NORM ? NS : 1], wv[NORM ? NS : 1], dv[NORM == 2 ? NS : 1], dwv[NORM == 2 ? NS : 1];
+    const int ux = NORM && NS > 1 ? (nks * 32 + 2047) >> 11 : 1, nslots = NORM ? (NS == 1 ? 1 : n * ux) : 0;
     if constexpr (NORM) {
+        static_assert(WV == 8, "a slot is 512 threads wide");
         int t = 0, u = 0;
 #pragma unroll
-        for (int s = 0; s < FEW_NORM_SLOTS; s++)
+        for (int s = 0; s < NS; s++)
             if (s < nslots) {
-                const int k = u * 512 + tid;
+                const int k = u * 2048 + tid * 4;
+                const bool in = k < P.ndim;
                 if constexpr (NORM == 2) {
-                    dv[s] = k < P.ndim ? P.nd[(long long)t * P.nld + k] : 0.f;
-                    dwv[s] = k < P.ndim ? P.ndw[k] : 0.f;
+                    dv[s] = in ? *reinterpret_cast<const f32x4 *>(P.nd + (long long)t * P.nld + k) : f32x4{};
+                    dwv[s] = in ? *reinterpret_cast<const f32x4 *>(P.ndw + k) : f32x4{};
                 }
-                xv[s] = k < P.ndim ? P.nx[(long long)t * P.nld + k] : 0.f;
-                wv[s] = k < P.ndim ? P.nw[k] : 0.f;
+                xv[s] = in ? *reinterpret_cast<const f32x4 *>(P.nx + (long long)t * P.nld + k) : f32x4{};
+                wv[s] = in ? *reinterpret_cast<const f32x4 *>(P.nw + k) : f32x4{};
                 if (++u == ux) { u = 0; t++; }
             }
     }
@@ -546,65 +653,51 @@ __global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P, TAIL tail) {
     load(w);
     T *xs = reinterpret_cast<T *>(lds);                    // NORM: [nks][4][n][8]
     if constexpr (NORM) {
-        float *red = reinterpret_cast<float *>(lds + (size_t)nks * 32 * n * sizeof(T));      // [n][WV]
-        int t = 0, u = 0;
-        float ss = 0.f;
-        if constexpr (NORM == 2) {
-            float *redd = red + n * WV;
+        float *red = reinterpret_cast<float *>(lds + (size_t)nks * 32 * n * sizeof(T));      // [NORM][n][WV]
+        auto sums = [&](const f32x4 *v, float *to) {         // every wavefront's sums of squares, per token
+            int t = 0, u = 0;
+            float ss = 0.f;
 #pragma unroll
-            for (int s = 0; s < FEW_NORM_SLOTS; s++)
+            for (int s = 0; s < NS; s++)
                 if (s < nslots) {
-                    ss += dv[s] * dv[s];
+                    ss += v[s][0] * v[s][0] + v[s][1] * v[s][1] + v[s][2] * v[s][2] + v[s][3] * v[s][3];
                     if (++u == ux) {
                         ss = wave_sum(ss);
-                        if (lane == 0) redd[t * WV + w] = ss;
+                        if (lane == 0) to[t * WV + w] = ss;
                         ss = 0.f; u = 0; t++;
                     }
                 }
             lds_barrier();
+        };
+        auto inverse = [&](const float *from, int t) {
+            const f32x4 q = *reinterpret_cast<const f32x4 *>(from + t * WV) + *reinterpret_cast<const f32x4 *>(from + t * WV + 4);
+            return rsqrt_f32(((q[0] + q[1]) + (q[2] + q[3])) / (float)P.ndim + P.neps);
+        };
+        if constexpr (NORM == 2) {
+            float *redd = red + n * WV;
+            sums(dv, redd);
             const bool keep = P.nxo && blockIdx.x == 0 && blockIdx.y == 0;
+            int t = 0, u = 0;
             float invd = 0.f;
-            t = u = 0;
 #pragma unroll
-            for (int s = 0; s < FEW_NORM_SLOTS; s++)
+            for (int s = 0; s < NS; s++)
                 if (s < nslots) {
-                    if (u == 0) {
-                        float q = 0.f;
-#pragma unroll
-                        for (int i = 0; i < WV; i++) q += redd[t * WV + i];
-                        invd = rsqrt_f32(q / (float)P.ndim + P.neps);
-                    }
+                    if (u == 0) invd = inverse(redd, t);
                     xv[s] += dv[s] * invd * dwv[s];
-                    const int k = u * 512 + tid;
-                    if (keep && k < P.ndim) P.nxo[(long long)t * P.nld + k] = xv[s];
+                    const int k = u * 2048 + tid * 4;
+                    if (keep && k < P.ndim) *reinterpret_cast<f32x4 *>(P.nxo + (long long)t * P.nld + k) = xv[s];
                     if (++u == ux) { u = 0; t++; }
                 }
-            t = u = 0;
         }
-#pragma unroll
-        for (int s = 0; s < FEW_NORM_SLOTS; s++)
-            if (s < nslots) {
-                ss += xv[s] * xv[s];
-                if (++u == ux) {
-                    ss = wave_sum(ss);
-                    if (lane == 0) red[t * WV + w] = ss;
-                    ss = 0.f; u = 0; t++;
-                }
-            }
-        lds_barrier();
+        sums(xv, red);
+        int t = 0, u = 0;
         float inv = 0.f;
-        t = u = 0;
 #pragma unroll
-        for (int s = 0; s < FEW_NORM_SLOTS; s++)
+        for (int s = 0; s < NS; s++)
             if (s < nslots) {
-                if (u == 0) {
-                    float q = 0.f;
-#pragma unroll
-                    for (int i = 0; i < WV; i++) q += red[t * WV + i];
-                    inv = rsqrt_f32(q / (float)P.ndim + P.neps);
-                }
-                const int k = u * 512 + tid;
-                if (k < nks * 32) put(xs + ((k >> 3) * n + t) * 8 + (k & 7), xv[s] * inv * wv[s]);
+                if (u == 0) inv = inverse(red, t);
+                const int k = u * 2048 + tid * 4;
+                if (k < nks * 32) put4(xs + ((k >> 3) * n + t) * 8 + (k & 7), xv[s] * inv * wv[s]);
                 if (++u == ux) { u = 0; t++; }
             }
         lds_barrier();
@@ -662,25 +755,27 @@ __global__ void __launch_bounds__(WV * 64) few_kernel(MatParams P, TAIL tail) {
     }
 }
 
-template <typename T, int EPI, int NT, int WV, int NORM, class TAIL>
+template <typename T, int EPI, int NT, int WV, int NORM, class TAIL, int NS = 1>
 hipError_t launch_few_nt(const MatParams &P, hipStream_t st, TAIL tail) {
     constexpr int RB = EPI == ST_GATED ? 2 : 1;
     const int tt = (P.n_tokens + 15) / 16;
     size_t lds = (size_t)WV * RB * NT * 64 * 16;           // at most 64 KB
     if (NORM) lds = std::max(lds, (size_t)P.nks * 32 * P.n_tokens * sizeof(T) + (size_t)P.n_tokens * WV * 4 * NORM);
-    hipLaunchKernelGGL((few_kernel<T, EPI, NT, WV, NORM, TAIL>), dim3(P.nrt / RB + (TAIL::on ? (tail.units + WV - 1) / WV : 0), (tt + NT - 1) / NT), dim3(WV * 64), lds, st, P, tail);
+    hipLaunchKernelGGL((few_kernel<T, EPI, NT, WV, NORM, NS, TAIL>), dim3(P.nrt / RB + (TAIL::on ? (tail.units + WV - 1) / WV : 0), (tt + NT - 1) / NT), dim3(WV * 64), lds, st, P, tail);
     return hipGetLastError();
 }
-// is the norm of the product's input computed inside the launch?
-inline bool few_norm_ok(int n, int nks) { return n * ((nks * 32 + 511) / 512) <= FEW_NORM_SLOTS; }
+// is the norm of the product's input (rows of dim values, ld apart) computed inside the launch?
+inline int few_norm_slots(int n, int nks) { return n * ((nks * 32 + 2047) / 2048); }
+inline bool few_norm_ok(int n, int nks, int dim, int ld) { return few_norm_slots(n, nks) <= FEW_NORM_SLOTS && (dim & 3) == 0 && (ld & 3) == 0; }
 
 template <typename T, int EPI, class TAIL>
 hipError_t launch_few(const MatParams &P, hipStream_t st, int norm, TAIL tail) {
     constexpr int RB = EPI == ST_GATED ? 2 : 1;
-    if constexpr (EPI != ST_HEADS)
-        if (norm == 2) return launch_few_nt<T, EPI, 1, 8, 2>(P, st, tail);
+    const bool one = few_norm_slots(P.n_tokens, P.nks) == 1;
+    if constexpr (EPI != ST_HEADS && EPI != ST_RESID)
+        if (norm == 2) return one ? launch_few_nt<T, EPI, 1, 8, 2, TAIL, 1>(P, st, tail) : launch_few_nt<T, EPI, 1, 8, 2, TAIL, FEW_NORM_SLOTS>(P, st, tail);
     if constexpr (EPI != ST_RESID)
-        if (norm) return launch_few_nt<T, EPI, 1, 8, 1>(P, st, tail);
+        if (norm) return one ? launch_few_nt<T, EPI, 1, 8, 1, TAIL, 1>(P, st, tail) : launch_few_nt<T, EPI, 1, 8, 1, TAIL, FEW_NORM_SLOTS>(P, st, tail);
     const int tt = (P.n_tokens + 15) / 16, blocks = P.nrt / RB;
     // few row tiles: sixteen wavefronts to a workgroup, and token tiles on workgroups of their own, until the chip is covered
     const bool deep = RB == 1 && blocks < 256 && P.nks >= 48;

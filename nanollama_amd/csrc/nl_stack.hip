@@ -353,7 +353,7 @@ hipError_t normed_product(nl_engine *e, MatParams P, const float *nw, const int 
     float *keep = last ? nullptr : e->xcur == e->x ? e->x2 : e->x;
     const int norm = e->pend ? 2 : 1;
     hipError_t s;
-    if (!rows && few_norm_ok(P.n_tokens, P.nks)) {
+    if (!rows && few_norm_ok(P.n_tokens, P.nks, e->c.dim, e->c.dim)) {
         P.nx = e->xcur; P.nw = nw; P.nd = e->delta; P.ndw = e->pend; P.nxo = keep; P.ndim = e->c.dim;
         s = launch_product<T, EPI>(P, e->stream, norm);
     } else {
@@ -410,7 +410,7 @@ hipError_t latent_mixer(nl_engine *e, const StepIn &s, const Run &R, const Layer
     H.ld = (s.decode ? L.nks : qt) * 32;
     H.col[1] = s.decode ? L.kvt * 32 : L.dimp;
     if (s.decode) { H.xq = e->xq; H.xq_nks = L.xq_nks(); }
-    if (few_norm_ok(s.n, L.uq.nks)) {
+    if (few_norm_ok(s.n, L.uq.nks, N.q_rank, L.proj.rows)) {
         P.nx = e->proj + L.tdq; P.nw = L.dqnorm; P.ndim = N.q_rank; P.nld = L.proj.rows;
         rc = store.units ? launch_product<T, ST_HEADS>(P, st, 1, store) : launch_product<T, ST_HEADS>(P, st, 1);
     } else {

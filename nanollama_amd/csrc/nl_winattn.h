@@ -100,25 +100,30 @@ __global__ void __launch_bounds__(256) win_prep_kernel(WinParams P) {
 __device__ __forceinline__ float exp2_f32(float x) { return __builtin_amdgcn_exp2f(x); }
 constexpr float LOG2E = 1.4426950408889634f;
 
-// keys per stage, stages in the LDS ring, 1 KiB pieces a wavefront fetches per stage (a stage holds at most 8 M of them)
-template <typename T, int M> struct WinGeom {
-    static constexpr int KT = sizeof(T) == 2 ? 64 : 32, NST = M <= 2 ? 4 : M <= 4 ? 3 : 2, PW = 2 * M;
+// keys per stage, 1 KiB pieces a wavefront fetches per stage, stages in the LDS ring, for at most NK key tiles and NV value tiles
+template <typename T, int NK, int NV> struct WinGeom {
+    static constexpr int KT = sizeof(T) == 2 ? 64 : 32, PW = ((KT / 16 * NK + KT / 32 * NV) * (int)sizeof(T) / 2 + 3) / 4, NST = PW <= 4 ? 4 : PW <= 8 ? 3 : 2;
 };
 
-// grid (tiles, heads); M bounds the key tiles (nks <= M) and value tiles (nvt <= 2 M), FULL: both are equal to their bound
-template <typename T, int M, bool FULL>
-__global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
-    constexpr int KT = WinGeom<T, M>::KT, UNIT = OPT * sizeof(T), NST = WinGeom<T, M>::NST, PW = WinGeom<T, M>::PW;
+// tiles x heads workgroups.  FULL: nks and nvt are NK and NV, else bounded by them.  Workgroups b, b + 8, ... run on one XCD: every XCD
+// takes a contiguous range of (head, tile), so that a head's keys stay in one L2, long tiles (late ones) beside short ones.
+template <typename T, int NK, int NV, bool FULL>
+__global__ void __launch_bounds__(256) win_attn_kernel(WinParams P, int ntiles) {
+    using G = WinGeom<T, NK, NV>;
+    constexpr int KT = G::KT, UNIT = OPT * sizeof(T), NST = G::NST, PW = G::PW;
     extern __shared__ __align__(16) char lds[];
-    const WinTile tl = P.tiles[blockIdx.x];
-    const int h = blockIdx.y, gk = h / (P.heads / P.kv_heads), tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, c = lane & 15;
-    const int nks = FULL ? M : P.nks, nvt = FULL ? 2 * M : P.nvt, qi = w * 16 + c, tok = tl.tok0 + min(qi, tl.nq - 1), qpos = tl.pos0 + min(qi, tl.nq - 1);
+    const int total = ntiles * P.heads, per = (total + 7) / 8, id = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+    if ((int)(blockIdx.x >> 3) >= per || id >= total) return;
+    const int h = id / ntiles, ti = id - h * ntiles;
+    const WinTile tl = P.tiles[ti & 1 ? ti >> 1 : ntiles - 1 - (ti >> 1)];
+    const int gk = h / (P.heads / P.kv_heads), tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, c = lane & 15;
+    const int nks = FULL ? NK : P.nks, nvt = FULL ? NV : P.nvt, qi = w * 16 + c, tok = tl.tok0 + min(qi, tl.nq - 1), qpos = tl.pos0 + min(qi, tl.nq - 1);
     const int win = P.window > 0 ? P.window : 0x7fffffff;
-    Frag<T> qf[M];
+    Frag<T> qf[NK];
     {
         const T *q = reinterpret_cast<const T *>(P.q) + ((long long)tok * P.heads + h) * nks * 32 + g * 8;
 #pragma unroll
-        for (int k = 0; k < M; k++)
+        for (int k = 0; k < NK; k++)
             if (FULL || k < nks) qf[k] = *reinterpret_cast<const Frag<T> *>(q + k * 32);
     }
     const char *K = reinterpret_cast<const char *>(ring_k<T>(P, tl.stream, gk)), *V = reinterpret_cast<const char *>(ring_v<T>(P, tl.stream, gk));
@@ -131,11 +136,11 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
         const char *ks = K + (long long)(slot >> 4) * nks * UNIT + lane * 16, *vs = V + (long long)(slot >> 5) * nvt * UNIT + lane * 16;
 #pragma unroll
         for (int i = 0; i < PW; i++) {                   // (the same number for every wavefront: pieces past the end repeat the last one)
-            const int u = FULL ? i * 4 + w : min(i * 4 + w, kpieces + vpieces - 1);
+            const int u = FULL && PW * 4 == (KT / 16 * NK + KT / 32 * NV) * (UNIT / 1024) ? i * 4 + w : min(i * 4 + w, kpieces + vpieces - 1);
             lds_dma16(u < kpieces ? ks + u * 1024 : vs + (u - kpieces) * 1024, lds + st * stage + u * 1024);
         }
     };
-    f32x4 o[2 * M] = {};
+    f32x4 o[NV] = {};
     float m = -INFINITY, l = 0.f;
     const float scale = P.scale * LOG2E, slope = P.slope ? P.slope[h] * LOG2E : 0.f;
     float off[KT / 16][4];                               // slope * (key's place in the tile)
@@ -157,7 +162,7 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
         const char *kb = lds + st * stage, *vb = kb + kpieces * 1024;
         f32x4 s[KT / 16] = {};
 #pragma unroll
-        for (int k = 0; k < M; k++)
+        for (int k = 0; k < NK; k++)
             if (FULL || k < nks) {
 #pragma unroll
                 for (int a = 0; a < KT / 16; a++)
@@ -199,7 +204,7 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
             }
         l = l * corr + add;
 #pragma unroll
-        for (int t = 0; t < 2 * M; t++)
+        for (int t = 0; t < NV; t++)
             if (FULL || t < nvt) {
                 o[t] *= corr;
 #pragma unroll
@@ -219,7 +224,7 @@ __global__ void __launch_bounds__(256) win_attn_kernel(WinParams P) {
     const float *gz = P.proj + (long long)tok * P.ldp + P.off_g + (P.head_gate ? h : h * P.dv);
     const int gs = P.head_gate ? 0 : 1;
 #pragma unroll
-    for (int t = 0; t < 2 * M; t++)
+    for (int t = 0; t < NV; t++)
         if (FULL || t < nvt) {
             const int d = t * 16 + 4 * g, k = P.y_k0 + h * P.dv + d;
             if (d + 3 < P.dv && (k & 3) == 0) {
@@ -474,16 +479,21 @@ hipError_t launch_win_attn(const WinParams &P, int ntiles, hipStream_t st) {
         // (more than 64 KB of LDS needs the attribute; cheap enough to set at every such launch)
         if (lds > 65536)
             if (hipError_t s = hipFuncSetAttribute(reinterpret_cast<const void *>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)) return s;
-        hipLaunchKernelGGL(kfn, dim3(ntiles, P.heads), dim3(256), lds, st, P);
+        hipLaunchKernelGGL(kfn, dim3((ntiles * P.heads + 7) / 8 * 8), dim3(256), lds, st, P, ntiles);
         return hipGetLastError();
     };
-    const int m = std::max(P.nks, (P.nvt + 1) / 2);
-    const bool full = P.nvt == 2 * P.nks;
-    if (m <= 1) return go(win_attn_kernel<T, 1, false>, WinGeom<T, 1>::NST);
-    if (m <= 2) return full && m == 2 ? go(win_attn_kernel<T, 2, true>, WinGeom<T, 2>::NST) : go(win_attn_kernel<T, 2, false>, WinGeom<T, 2>::NST);
-    if (m <= 3) return go(win_attn_kernel<T, 3, false>, WinGeom<T, 3>::NST);
-    if (m <= 4) return full && m == 4 ? go(win_attn_kernel<T, 4, true>, WinGeom<T, 4>::NST) : go(win_attn_kernel<T, 4, false>, WinGeom<T, 4>::NST);
-    return go(win_attn_kernel<T, 8, false>, WinGeom<T, 8>::NST);
+    const int k = P.nks, v = P.nvt;
+#define NL_WIN(NK, NV, FULL) return go(win_attn_kernel<T, NK, NV, FULL>, WinGeom<T, NK, NV>::NST)
+    // sizes of their own: 64 / 64, 64 + 32 / 64, 128 / 128, 128 + 64 / 128
+    if (k == 2 && v == 4) NL_WIN(2, 4, true);
+    if (k == 3 && v == 4) NL_WIN(3, 4, true);
+    if (k == 4 && v == 8) NL_WIN(4, 8, true);
+    if (k == 6 && v == 8) NL_WIN(6, 8, true);
+    if (k <= 1 && v <= 2) NL_WIN(1, 2, false);
+    if (k <= 2 && v <= 4) NL_WIN(2, 4, false);
+    if (k <= 4 && v <= 8) NL_WIN(4, 8, false);
+    NL_WIN(8, 16, false);
+#undef NL_WIN
 }
 
 }  // namespace nl
