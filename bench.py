@@ -686,7 +686,7 @@ def stack_sizes(design="ganidra"):
     return out
 
 
-def time_model(dev, vocab, streams, phases, prompt_len=2047, pos=512, steps=128, batch_steps=32):
+def time_model(dev, vocab, streams, phases, prompt_len=2047, pos=512, steps=128, batch_steps=32, batch_pos=64):
     """Prompt, single-stream greedy decode and a batch of decode streams of one loaded model (host wall clock, best of three)."""
     import numpy as np
     from nanollama_amd import synth
@@ -727,8 +727,8 @@ def time_model(dev, vocab, streams, phases, prompt_len=2047, pos=512, steps=128,
         ids = list(range(streams))
         for s in ids:
             dev.reset(s)
-            dev.prefill(toks[:64], 0, s, want_logits=False)
-        at = [64]
+            dev.prefill(toks[:batch_pos], 0, s, want_logits=False)
+        at = [batch_pos]
 
         def batch(n):
             for _ in range(n):
@@ -736,11 +736,11 @@ def time_model(dev, vocab, streams, phases, prompt_len=2047, pos=512, steps=128,
                 at[0] += 1
         batch(4)
         dt = best(lambda: batch(batch_steps)) / batch_steps
-        out.update(batch_streams=streams, batch_ms_per_step=round(dt * 1e3, 4), batch_tokens_per_s=round(streams / dt))
+        out.update(batch_streams=streams, batch_position=batch_pos, batch_ms_per_step=round(dt * 1e3, 4), batch_tokens_per_s=round(streams / dt))
     return out
 
 
-def stack_bench(names, only=None, phases=("prefill", "decode", "batch"), design="ganidra"):
+def stack_bench(names, only=None, phases=("prefill", "decode", "batch"), design="ganidra", batch_pos=64):
     """A layer-stack design (bfloat16) beside the quantised family's F16 files of equal size; random weights."""
     from nanollama_amd import _lib, gguf, model, synth_stack
     from nanollama_amd.designs import DESIGNS
@@ -753,13 +753,13 @@ def stack_bench(names, only=None, phases=("prefill", "decode", "batch"), design=
             w = (synth_stack.pabalix_weights if design == "pabalix" else synth_stack.ganidra_weights)(cfg, 1, fast=True)
             spec = DESIGNS[cfg["architecture"]](cfg, lambda n: w[n].shape)
             dev = load_stack_model(spec, lambda n: ("BF16", w[n]), max_streams=64, seq_len=4096)
-            r[design + "_bf16"] = dict(time_model(dev, shape.vocab, 64, phases), params_millions=dev.config.num_params // 1000000)
+            r[design + "_bf16"] = dict(time_model(dev, shape.vocab, 64, phases, batch_pos=batch_pos), params_millions=dev.config.num_params // 1000000)
             dev.close()
             del w
         if only in (None, "llama"):
             g = gguf.load_gguf(ensure_gguf(shape, "f16", "float"))
             dev = model.load_llama_model(g, max_streams=64)
-            r["llama_f16"] = dict(time_model(dev, shape.vocab, 64, phases), params_millions=(shape.matrix_params() + shape.vocab * shape.dim) // 1000000)
+            r["llama_f16"] = dict(time_model(dev, shape.vocab, 64, phases, batch_pos=batch_pos), params_millions=(shape.matrix_params() + shape.vocab * shape.dim) // 1000000)
             dev.close()
         res[name] = r
         print(f"[bench] {name}: {json.dumps(r)}", file=sys.stderr, flush=True)
@@ -808,11 +808,13 @@ def main():
     ap.add_argument("--stack", nargs="?", const="mini,goldie,wide", default=None, metavar="SIZES",
                     help="one GPU: time the layer-stack design beside an F16 Llama of equal size and print that line only")
     ap.add_argument("--stack-design", choices=("ganidra", "pabalix"), default="ganidra", help="with --stack: which layer-stack design")
+    ap.add_argument("--stack-context", type=int, default=64, help="with --stack: position of the batch's streams (up to 1900)")
     ap.add_argument("--stack-only", choices=("stack", "llama"), default=None, help="with --stack: one of the two models")
     ap.add_argument("--stack-phase", choices=("prefill", "decode", "batch"), default=None, help="with --stack: one of the three measurements (profiling)")
     args = ap.parse_args()
     if args.stack:
-        print(json.dumps(stack_bench(args.stack.split(","), args.stack_only, (args.stack_phase,) if args.stack_phase else ("prefill", "decode", "batch"), args.stack_design)))
+        print(json.dumps(stack_bench(args.stack.split(","), args.stack_only, (args.stack_phase,) if args.stack_phase else ("prefill", "decode", "batch"), args.stack_design,
+                                     min(max(args.stack_context, 1), 1900))))
         return
     n = args.gpus
     if n < 1:

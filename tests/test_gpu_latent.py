@@ -115,6 +115,49 @@ def test_sizes(name, dtype):
     m.close()
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("width", [50, 516, 1030, 1100, 2052, 4100, 8200])
+def test_norms_of_every_width_and_row_count(width, dtype):
+    """The norms (with and without a pending sublayer) run inside a product, a row per workgroup, several rows per workgroup or in
+    pieces, by width and tokens: prompts of 300, 200 and 65, decode batches of 1 to 6."""
+    cfg = lconfig([lat(1, ff=20), lat(3, q_rank=36), lat(2, q_rank=2 * (width // 4) + 1 if width < 2000 else 40)], width=width)
+    w = weights(cfg, 13)
+    fl = floats(w)
+    m = load(cfg, w, dtype, max_streams=7, seq_len=320)
+    ids = tokens(306, seed=7)
+    want = so.forward(cfg, fl, ids)
+    tol = bound(dtype, cfg, fl, ids, want)
+    places = [0, 7, 8, 15, 63, 64, 190, 255, 256, 299]
+    assert rel(whole(m, ids[:300], places), want[places]) < tol
+    for n, st in ((200, 1), (65, 2), (64, 3), (17, 4), (3, 5)):
+        assert rel(whole(m, ids[:n], None, st), want[:n]) < tol, n
+    at = [300, 200, 65, 64, 17, 3]
+    for n in (6, 5, 4, 3, 2, 1):
+        out = m.step([(st, [ids[at[st]]], at[st], [0]) for st in range(n)])
+        for st, o in enumerate(out):
+            assert rel(o, want[at[st]]) < tol, (n, st)
+            at[st] += 1
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("dim,rot,vdim", [(8, 4, 32), (24, 20, 64), (64, 24, 64), (90, 30, 128), (128, 64, 128), (40, 64, 80), (190, 60, 240)])
+def test_long_prompts_at_every_head_size_of_the_prompt_attention(dim, rot, vdim, dtype):
+    cfg = lconfig([lat(3, heads=3, dim=dim, rot=rot, vdim=vdim, yarn=YARN), lat(2, heads=2, dim=dim, rot=rot, vdim=vdim)])
+    w = weights(cfg, 17)
+    fl = floats(w)
+    ids, other = tokens(430, seed=8), tokens(150, seed=9)
+    want, want2 = so.forward(cfg, fl, ids), so.forward(cfg, fl, other)
+    tol = bound(dtype, cfg, fl, ids, want)
+    m = load(cfg, w, dtype, max_streams=2, seq_len=430)
+    assert rel(whole(m, ids), want) < tol
+    m.step([(0, ids[:100], 0, []), (1, other[:33], 0, [])])
+    a, b = m.step([(0, ids[100:350], 100, list(range(250))), (1, other[33:], 33, list(range(117)))])
+    assert rel(a, want[100:350]) < tol and rel(b, want2[33:]) < tol
+    assert rel(by_token(m, ids[350:360], 0, 350), want[350:360]) < tol
+    m.close()
+
+
 # ---- cuts, batches, slots -------------------------------------------------------------------------------------------------------
 
 @pytest.fixture(scope="module")
